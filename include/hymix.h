@@ -6,7 +6,8 @@
  * sinks and sliding windows that keep the first tokens, the generalized delta rule with a float32 state per
  * sequence, and squared ReLU.  Later additions: the grouped-norm and the Dynamic-Tanh residual boundaries, pooled
  * blocks, chunked masks and sigmoid weights in the attention kernels, interleaved rotation on any frequency table and
- * unit-RMS value heads in the preparation, and linear attention with a constant decay per head and a float32 state.
+ * unit-RMS value heads in the preparation, linear attention with a constant decay per head and a float32 state, the
+ * layer-norm residual boundary, and the selective scan.
  *
  * Conventions (those of libqlinear and libseqmix): all pointers are DEVICE pointers owned by the caller,
  * matrices are row-major and dense unless a stride (in elements) is named; `stream` is a hipStream_t passed as
@@ -64,8 +65,9 @@ int hm_token_shift(int dtype, const void* h, const void* mu, const void* state, 
                    const int32_t* tok_pos, const int32_t* qstart, const int32_t* seq_slot, void* out, int64_t T, int W,
                    void* stream);
 
-/* out[t, c] = max(z[t, c], 0)^2; z rows are z_stride elements apart. */
-int hm_relu_squared(int dtype, const void* z, int64_t z_stride, void* out, int64_t T, int F, void* stream);
+/* out[t, c] = row_scale[t] * max(z[t, c], 0)^2 (row_scale f32 [T], NULL = 1); rows are z_stride and out_stride elements apart. */
+int hm_relu_squared(int dtype, const void* z, int64_t z_stride, const float* row_scale, void* out, int64_t out_stride, int64_t T,
+                    int F, void* stream);
 
 /* qkv [T, H*D + G*D + G*V] (rows row_stride apart), per token:
  *   q_norm_w / k_norm_w != NULL: RMS norm over the whole q (k) projection with that weight;
@@ -170,6 +172,28 @@ int hm_dyt_residual(int dtype, float* x, const void* y, const int64_t* ids, cons
  *   h_out != NULL:           h_out[t] = next_w ? group_norm(x[t]) * next_w : x[t], in the storage type. */
 int hm_group_norm_residual(int dtype, float* x, const void* y, const int64_t* ids, const void* post_w, const void* next_w,
                            int groups, float eps, void* h_out, int64_t T, int W, void* stream);
+
+/* The boundary between two blocks of a residual whose blocks read a layer norm of it (weight, no bias); x [T, W] f32 is updated
+ * in place, per token in one launch:
+ *   y != NULL, ids == NULL:  x[t] += y[t]
+ *   y != NULL, ids != NULL:  x[t]  = y[ids[t]]                            (y = an embedding table)
+ *   y2 != NULL:              x[t] += y2[t]
+ *   prod != NULL:            x[t] += sum_{k < top} wts[t * top + k] * prod[pair_row[t * top + k]]   (wts NULL = 1; the per-pair
+ *                            rows that sm_moe_grouped / sm_moe_tiles128 leave with y = NULL)
+ *   h_out != NULL:           h_out[t] = (x[t] - m) / sqrt(mean((x[t] - m)^2) + eps) * next_w, m = mean(x[t]), in the storage type. */
+int hm_layer_norm_residual(int dtype, float* x, const void* y, const int64_t* ids, const void* y2, const void* prod,
+                           const int32_t* pair_row, const float* wts, int top, const void* next_w, float eps, void* h_out,
+                           int64_t T, int W, void* stream);
+
+/* Selective scan.  x, z [T, C] and bc (columns b_off, c_off: B, C of N states) in the storage type, dt_pre f32 [T, C], all with
+ * row strides; A f32 [C, N], dt_bias, D f32 [C].  For every sequence b and channel c, over the tokens of its portion in order:
+ *   dt = softplus(dt_pre + dt_bias);  S[n] <- exp(dt A[c, n]) S[n] + dt x B[n];  out = (sum_n S[n] C[n] + D x) * silu(z)
+ * state f32 [slots, C, N] is read at the start unless seq_pos0[b] == 0 (then S = 0) and written at the end.  out [T, C] rows
+ * out_stride apart, in the storage type.  N <= 512.  max_q = the longest portion of the step (a hint for staging only). */
+int hm_selective_scan(int dtype, const void* x, int64_t x_stride, const float* dt_pre, int64_t dt_stride, const float* dt_bias,
+                      const void* bc, int64_t bc_stride, int b_off, int c_off, const float* A, const float* D, const void* z,
+                      int64_t z_stride, float* state, const int32_t* qstart, const int32_t* seq_pos0, const int32_t* seq_slot,
+                      void* out, int64_t out_stride, int B, int C, int N, int max_q, void* stream);
 
 /* x[i] <- cap * tanh(x[i] * scale / cap) (cap <= 0: x[i] * scale), f32 in place. */
 int hm_scale_softcap(float* x, int64_t n, float scale, float cap, void* stream);

@@ -105,11 +105,13 @@ __global__ void token_shift_kernel(const T* __restrict__ h, const T* __restrict_
 }
 
 template <typename T>
-__global__ void relu_squared_kernel(const T* __restrict__ z, int64_t z_stride, T* __restrict__ out, int F) {
+__global__ void relu_squared_kernel(const T* __restrict__ z, int64_t z_stride, const float* __restrict__ row_scale,
+                                    T* __restrict__ out, int64_t out_stride, int F) {
     const int64_t t = blockIdx.x;
+    const float rs = row_scale ? row_scale[t] : 1.f;
     for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < F; c += gridDim.y * blockDim.x) {
         const float v = fmaxf(to_f(z[(size_t)t * z_stride + c]), 0.f);
-        out[(size_t)t * F + c] = from_f<T>(v * v);
+        out[(size_t)t * out_stride + c] = from_f<T>(rs * (v * v));
     }
 }
 
@@ -173,13 +175,14 @@ extern "C" int hm_token_shift(int dtype, const void* h, const void* mu, const vo
     return HM_OK;
 }
 
-extern "C" int hm_relu_squared(int dtype, const void* z, int64_t z_stride, void* out, int64_t T, int F, void* stream) {
-    if (T < 0 || F < 1 || z_stride < F || (T > 0 && (!z || !out))) { set_error("hm_relu_squared: bad argument"); return HM_EINVAL; }
+extern "C" int hm_relu_squared(int dtype, const void* z, int64_t z_stride, const float* row_scale, void* out, int64_t out_stride,
+                               int64_t T, int F, void* stream) {
+    if (T < 0 || F < 1 || z_stride < F || out_stride < F || (T > 0 && (!z || !out))) { set_error("hm_relu_squared: bad argument"); return HM_EINVAL; }
     if (T == 0) return HM_OK;
     dim3 grid((unsigned)T, (unsigned)((F + 1023) / 1024));
     HM_DISPATCH(dtype, "hm_relu_squared",
                 hipLaunchKernelGGL(relu_squared_kernel<DT>, grid, dim3(256), 0, as_stream(stream), (const DT*)z, z_stride,
-                                   (DT*)out, F));
+                                   row_scale, (DT*)out, out_stride, F));
     HM_CHECK_LAUNCH("hm_relu_squared");
     return HM_OK;
 }

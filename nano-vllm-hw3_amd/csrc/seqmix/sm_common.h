@@ -43,21 +43,27 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
     return t;
 }
 
-// what an expert applies between its two products (SM_ACT_*): the clamped GLU of a gate and an up product, or a GELU
-// of the up product alone (exact, or the tanh form)
+// what a feed-forward applies between its two products (SM_ACT_*): a gated form of a gate and an up product (clamped GLU,
+// SiLU or tanh-GELU gate), or a function of the up product alone (exact or tanh GELU, squared ReLU)
 __device__ __forceinline__ float gelu_erf(float z) { return 0.5f * z * (1.f + erff(z * 0.70710678118654752f)); }
 __device__ __forceinline__ float gelu_tanh(float z) {
     return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
 // the gated forms: g' = min(g, limit), u' = clamp(u, +-limit), g' sigmoid(alpha g') (u' + 1) (SM_ACT_CLAMPED_GLU), or with
-// SM_ACT_SILU_GLU the same without the one: silu(g) u for limit = +inf and alpha = 1
+// SM_ACT_SILU_GLU the same without the one: silu(g) u for limit = +inf and alpha = 1; SM_ACT_GELU_TANH_GLU: gelu_tanh(g) u
 __device__ __forceinline__ float gated_act(float g, float u, float limit, float alpha, int act) {
+    if (act == SM_ACT_GELU_TANH_GLU) return gelu_tanh(g) * u;
     g = fminf(g, limit);
     u = fminf(fmaxf(u, -limit), limit);
     return g / (1.f + __expf(-alpha * g)) * (u + (act == SM_ACT_SILU_GLU ? 0.f : 1.f));
 }
-__device__ __forceinline__ bool act_is_gated(int act) { return act == SM_ACT_CLAMPED_GLU || act == SM_ACT_SILU_GLU; }
-__device__ __forceinline__ float plain_act(float z, int act) { return act == SM_ACT_GELU_TANH ? gelu_tanh(z) : gelu_erf(z); }
+__host__ __device__ __forceinline__ bool act_is_gated(int act) {
+    return act == SM_ACT_CLAMPED_GLU || act == SM_ACT_SILU_GLU || act == SM_ACT_GELU_TANH_GLU;
+}
+__device__ __forceinline__ float plain_act(float z, int act) {
+    if (act == SM_ACT_RELU_SQ) { z = fmaxf(z, 0.f); return z * z; }
+    return act == SM_ACT_GELU_TANH ? gelu_tanh(z) : gelu_erf(z);
+}
 
 static inline hipStream_t as_stream(void* s) { return (hipStream_t)s; }
 

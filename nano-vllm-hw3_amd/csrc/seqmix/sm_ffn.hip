@@ -1,4 +1,5 @@
-// Activations of the feed-forward layers: PolyNorm (a normalised cubic polynomial of a row) and the clamped GLU.
+// Activations of the feed-forward layers: PolyNorm (a normalised cubic polynomial of a row), the clamped GLU and the other
+// gated forms.
 #include "sm_common.h"
 
 namespace sm {
@@ -39,26 +40,21 @@ __global__ __launch_bounds__(256) void poly_norm_kernel(const T* __restrict__ z,
     }
 }
 
-__device__ __forceinline__ float clamped_glu(float g, float u, float limit, float alpha) {
-    g = fminf(g, limit);
-    u = fminf(fmaxf(u, -limit), limit);
-    return g / (1.f + __expf(-alpha * g)) * (u + 1.f);
-}
-
-// VEC consecutive columns per thread (VEC = 8 when F % 8 == 0: whole 16-byte accesses for bf16)
+// VEC consecutive columns per thread (VEC = 8 where rows allow: whole 16-byte accesses for bf16)
 template <typename T, int VEC>
-__global__ void clamped_glu_kernel(const T* __restrict__ gu, float limit, float alpha, T* __restrict__ out, int64_t n, int F) {
+__global__ void gated_act_kernel(const T* __restrict__ gu, int64_t row_stride, int act, float limit, float alpha,
+                                 T* __restrict__ out, int64_t out_stride, int64_t n, int F) {
     const int64_t i = ((int64_t)blockIdx.x * blockDim.x + threadIdx.x) * VEC;
     if (i >= n) return;
     const int64_t t = i / F;
     const int c = (int)(i - t * F);
-    const T* row = gu + (size_t)t * 2 * F;
+    const T* row = gu + (size_t)t * row_stride;
     struct alignas(sizeof(T) * VEC) Pack { T v[VEC]; };
     const Pack g = *(const Pack*)(row + c), u = *(const Pack*)(row + F + c);
     Pack o;
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) o.v[e] = from_f<T>(clamped_glu(to_f(g.v[e]), to_f(u.v[e]), limit, alpha));
-    *(Pack*)(out + i) = o;
+    for (int e = 0; e < VEC; ++e) o.v[e] = from_f<T>(gated_act(to_f(g.v[e]), to_f(u.v[e]), limit, alpha, act));
+    *(Pack*)(out + (size_t)t * out_stride + c) = o;
 }
 
 }  // namespace sm
@@ -79,17 +75,25 @@ extern "C" int sm_poly_norm(int dtype, const void* z, const float* coef, float e
     return SM_OK;
 }
 
-extern "C" int sm_clamped_glu(int dtype, const void* gu, float limit, float alpha, void* out, int64_t T, int F, void* stream) {
-    if (T < 0 || F < 1 || (T > 0 && (!gu || !out))) { set_error("sm_clamped_glu: bad argument"); return SM_EINVAL; }
+extern "C" int sm_gated_act(int dtype, const void* gu, int64_t row_stride, int act_kind, float limit, float alpha, void* out,
+                            int64_t out_stride, int64_t T, int F, void* stream) {
+    if (T < 0 || F < 1 || row_stride < 2 * (int64_t)F || out_stride < F || !act_is_gated(act_kind) || (T > 0 && (!gu || !out))) {
+        set_error("sm_gated_act: bad argument");
+        return SM_EINVAL;
+    }
     if (T == 0) return SM_OK;
     const int64_t n = T * F;
-    SM_DISPATCH(dtype, "sm_clamped_glu",
-                if (F % 8 == 0)
-                    hipLaunchKernelGGL((clamped_glu_kernel<DT, 8>), dim3((unsigned)((n / 8 + 255) / 256)), dim3(256), 0,
-                                       as_stream(stream), (const DT*)gu, limit, alpha, (DT*)out, n, F);
-                else
-                    hipLaunchKernelGGL((clamped_glu_kernel<DT, 1>), dim3((unsigned)((n + 255) / 256)), dim3(256), 0,
-                                       as_stream(stream), (const DT*)gu, limit, alpha, (DT*)out, n, F));
-    SM_CHECK_LAUNCH("sm_clamped_glu");
+    const bool wide = F % 8 == 0 && row_stride % 8 == 0 && out_stride % 8 == 0 && ((uintptr_t)gu | (uintptr_t)out) % 16 == 0;
+#define SM_GLU(VEC_)                                                                                                            \
+    hipLaunchKernelGGL((gated_act_kernel<DT, VEC_>), dim3((unsigned)((n / VEC_ + 255) / 256)), dim3(256), 0, as_stream(stream), \
+                       (const DT*)gu, row_stride, act_kind, limit, alpha, (DT*)out, out_stride, n, F)
+    SM_DISPATCH(dtype, "sm_gated_act", if (wide) SM_GLU(8); else SM_GLU(1));
+#undef SM_GLU
+    SM_CHECK_LAUNCH("sm_gated_act");
     return SM_OK;
+}
+
+extern "C" int sm_clamped_glu(int dtype, const void* gu, float limit, float alpha, void* out, int64_t T, int F, void* stream) {
+    if (F < 1) { set_error("sm_clamped_glu: bad argument"); return SM_EINVAL; }
+    return sm_gated_act(dtype, gu, 2 * (int64_t)F, SM_ACT_CLAMPED_GLU, limit, alpha, out, F, T, F, stream);
 }

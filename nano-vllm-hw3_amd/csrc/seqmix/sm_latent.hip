@@ -28,26 +28,33 @@ __global__ __launch_bounds__(64) void latent_norm_store_kernel(const T* __restri
 // The latent with a rotated key part beside it.  x rows hold [R latent | Rd key part]; the latent is RMS-normalised
 // with a weight, the first rot_dims channels of the key part turn by position * inv_freq (channel 2i pairs with 2i + 1),
 // and both are stored as one cache row [R + Rd].  The queries' own rotated parts (q rows hold per head [D | Rd]) turn
-// the same way and land in columns R .. R + Rd of the absorbed queries qa [T, H, R + Rd].  Angles are f32.
+// the same way and land in columns R .. R + Rd of the absorbed queries qa [T, H, R + Rd].  Angles are f32; rot_mag multiplies
+// every cosine and sine.  Without x only the queries are turned (the layer reads rows that another layer stored).
 template <typename T>
 __global__ __launch_bounds__(256) void latent_rope_store_kernel(const T* __restrict__ x, int64_t x_stride, const T* __restrict__ w,
                                                                 float eps, const T* __restrict__ q, int64_t q_stride,
                                                                 T* __restrict__ qa, const float* __restrict__ inv_freq,
                                                                 int rot_half, const int32_t* __restrict__ tok_pos,
                                                                 T* __restrict__ cache, const int32_t* __restrict__ slot_mapping,
-                                                                int H, int D, int R, int Rd) {
+                                                                int H, int D, int R, int Rd, float rot_mag) {
     extern __shared__ float cs[];              // rot_half cosines, then rot_half sines
     __shared__ float red[16];
     const int64_t t = blockIdx.x;
     const int tid = threadIdx.x, RK = R + Rd;
     const float pos = (float)tok_pos[t];
-    for (int i = tid; i < rot_half; i += 256) sincosf(pos * inv_freq[i], cs + rot_half + i, cs + i);
+    for (int i = tid; i < rot_half; i += 256) {
+        float sn, cn;
+        sincosf(pos * inv_freq[i], &sn, &cn);
+        cs[rot_half + i] = sn * rot_mag;
+        cs[i] = cn * rot_mag;
+    }
     const T* xr = x + (size_t)t * x_stride;
     float ss = 0.f;
-    for (int c = tid; c < R; c += 256) {
-        const float v = to_f(xr[c]);
-        ss += v * v;
-    }
+    if (x != nullptr)
+        for (int c = tid; c < R; c += 256) {
+            const float v = to_f(xr[c]);
+            ss += v * v;
+        }
     ss = block_sum(ss, red);                   // (its barriers also publish cs)
     const float r = 1.f / sqrtf(ss / (float)R + eps);
     // queries: head hd's rotated part
@@ -62,6 +69,7 @@ __global__ __launch_bounds__(256) void latent_rope_store_kernel(const T* __restr
         }
         qa[((size_t)t * H + hd) * RK + R + c] = from_f<T>(v);
     }
+    if (x == nullptr) return;
     const int slot = slot_mapping[t];
     if (slot < 0) return;
     T* out = cache + (size_t)slot * RK;
@@ -85,7 +93,7 @@ __global__ __launch_bounds__(256) void latent_attn_rows_kernel(const T* __restri
                                                                const int32_t* __restrict__ tok_seq,
                                                                const int32_t* __restrict__ tok_pos, T* __restrict__ o,
                                                                float scale, int H, int R, int block_size, int max_blocks,
-                                                               int RV, int window) {
+                                                               int RV, int window, const float* __restrict__ sink) {
     extern __shared__ float q_lds[];                 // R floats
     __shared__ float s_lds[kRowChunk];
     __shared__ int row_lds[kRowChunk];
@@ -138,7 +146,11 @@ __global__ __launch_bounds__(256) void latent_attn_rows_kernel(const T* __restri
         m_run = mx;
     }
     T* orow = o + ((size_t)t * H + hd) * RV;
-    const float inv = 1.f / l_run;
+    float inv = 1.f / l_run;
+    if (sink != nullptr) {                           // one more term of the denominator, without a key and a value
+        const float mx = fmaxf(m_run, sink[hd]), f = __expf(m_run - mx);
+        inv = f / (l_run * f + __expf(sink[hd] - mx));
+    }
     for (int r = 0; r < 4; ++r) {
         const int c = tid + 256 * r;
         if (c < RV) orow[c] = from_f<T>(acc[r] * inv);
@@ -179,7 +191,8 @@ extern "C" int sm_rms_norm_rows(int dtype, const void* x, int64_t row_stride, co
 
 extern "C" int sm_latent_attn_rows(int dtype, const void* q, const void* cache, const int32_t* block_tables,
                                    const int32_t* tok_seq, const int32_t* tok_pos, void* o, float scale, int64_t T, int H,
-                                   int R, int block_size, int max_blocks, int RV, int window, void* stream) {
+                                   int R, int block_size, int max_blocks, int RV, int window, const float* sink,
+                                   void* stream) {
     if (RV <= 0) RV = R;
     if (T < 0 || H < 1 || R < 1 || RV > R || window < 0 || block_size < 1 || max_blocks < 1 ||
         (T > 0 && (!q || !cache || !block_tables || !tok_seq || !tok_pos || !o))) {
@@ -192,7 +205,7 @@ extern "C" int sm_latent_attn_rows(int dtype, const void* q, const void* cache, 
     SM_DISPATCH(dtype, "sm_latent_attn_rows",
                 hipLaunchKernelGGL(latent_attn_rows_kernel<DT>, grid, dim3(256), (size_t)R * 4, as_stream(stream), (const DT*)q,
                                    (const DT*)cache, block_tables, tok_seq, tok_pos, (DT*)o, scale, H, R, block_size, max_blocks,
-                                   RV, window));
+                                   RV, window, sink));
     SM_CHECK_LAUNCH("sm_latent_attn_rows");
     return SM_OK;
 }
@@ -200,10 +213,10 @@ extern "C" int sm_latent_attn_rows(int dtype, const void* q, const void* cache, 
 extern "C" int sm_latent_rope_store(int dtype, const void* x, int64_t x_stride, const void* w, float eps, const void* q,
                                     int64_t q_stride, void* qa, const float* inv_freq, int rot_dims, const int32_t* tok_pos,
                                     void* cache, const int32_t* slot_mapping, int64_t T, int H, int D, int R, int Rd,
-                                    void* stream) {
-    if (T < 0 || H < 1 || D < 0 || R < 1 || Rd < 0 || rot_dims < 0 || rot_dims % 2 || rot_dims > Rd || x_stride < R + Rd ||
+                                    float rot_mag, void* stream) {
+    if (T < 0 || H < 1 || D < 0 || R < 1 || Rd < 0 || rot_dims < 0 || rot_dims % 2 || rot_dims > Rd || (x && x_stride < R + Rd) ||
         q_stride < (int64_t)H * (D + Rd) || (rot_dims > 0 && !inv_freq) ||
-        (T > 0 && (!x || !w || !q || !qa || !tok_pos || !cache || !slot_mapping))) {
+        (T > 0 && (!q || !qa || !tok_pos || (x && (!w || !cache || !slot_mapping))))) {
         set_error("sm_latent_rope_store: bad argument");
         return SM_EINVAL;
     }
@@ -212,7 +225,7 @@ extern "C" int sm_latent_rope_store(int dtype, const void* x, int64_t x_stride, 
     SM_DISPATCH(dtype, "sm_latent_rope_store",
                 hipLaunchKernelGGL(latent_rope_store_kernel<DT>, dim3((unsigned)T), dim3(256), (size_t)rot_dims * 4 + 16,
                                    as_stream(stream), (const DT*)x, x_stride, (const DT*)w, eps, (const DT*)q, q_stride, (DT*)qa,
-                                   inv_freq, rot_dims / 2, tok_pos, (DT*)cache, slot_mapping, H, D, R, Rd));
+                                   inv_freq, rot_dims / 2, tok_pos, (DT*)cache, slot_mapping, H, D, R, Rd, rot_mag));
     SM_CHECK_LAUNCH("sm_latent_rope_store");
     return SM_OK;
 }

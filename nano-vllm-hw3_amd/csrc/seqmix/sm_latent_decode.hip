@@ -48,7 +48,7 @@ __global__ __launch_bounds__(64 * WAVES) void latent_attn_decode_kernel(const un
 }
 
 __global__ void latent_decode_merge_kernel(const float* __restrict__ ws, unsigned short* __restrict__ o, int H, int R, int splits,
-                                           int stride) {
+                                           int stride, const float* __restrict__ sink) {
     const size_t row = blockIdx.x;                          // b * H + h
     const size_t b = row / H, h = row % H;
     float M = -INFINITY;
@@ -61,7 +61,7 @@ __global__ void latent_decode_merge_kernel(const float* __restrict__ ws, unsigne
         const float* p = ws + ((b * splits + s) * H + h) * stride;
         if (p[1] > 0.f) L += __builtin_amdgcn_exp2f(p[0] - M) * p[1];
     }
-    const float inv = 1.f / L;
+    const float inv = sink ? sink_inv(M, L, sink[h]) : 1.f / L;
     for (int c = threadIdx.x; c < R; c += blockDim.x) {
         float acc = 0.f;
         for (int s = 0; s < splits; ++s) {
@@ -93,7 +93,8 @@ extern "C" size_t sm_latent_decode_workspace_bytes(int64_t B, int H, int R, int 
 
 extern "C" int sm_latent_attn_decode(const void* q, const void* cache, const int32_t* block_tables, const int32_t* ctx, void* o,
                                      float scale, int64_t B, int H, int R, int block_size, int max_blocks, int splits,
-                                     void* workspace, size_t workspace_bytes, int RV, int window, void* stream) {
+                                     void* workspace, size_t workspace_bytes, int RV, int window, const float* sink,
+                                     void* stream) {
     if (RV <= 0) RV = R;
     if (B < 0 || H < 1 || R < 1 || RV > R || window < 0 || block_size < 1 || max_blocks < 1 || splits < 1 ||
         (B > 0 && (!q || !cache || !block_tables || !ctx || !o || !workspace))) {
@@ -123,7 +124,7 @@ extern "C" int sm_latent_attn_decode(const void* q, const void* cache, const int
 #undef SM_DEC
     SM_CHECK_LAUNCH("sm_latent_attn_decode");
     hipLaunchKernelGGL(latent_decode_merge_kernel, dim3((unsigned)(B * H)), dim3(64), 0, s, (const float*)workspace,
-                       (unsigned short*)o, H, RV, splits, part_stride(padded_nbv(R, RV)));
+                       (unsigned short*)o, H, RV, splits, part_stride(padded_nbv(R, RV)), sink);
     SM_CHECK_LAUNCH("sm_latent_attn_decode (merge)");
     return SM_OK;
 }

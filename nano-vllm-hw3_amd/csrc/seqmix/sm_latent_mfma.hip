@@ -12,7 +12,8 @@ __global__ __launch_bounds__(256) void latent_attn_tiles_kernel(const unsigned s
                                                                 const int32_t* __restrict__ qstart,
                                                                 const int32_t* __restrict__ seq_pos0,
                                                                 unsigned short* __restrict__ o, float c_log2, int H, int R,
-                                                                int block_size, int max_blocks, int RV, int window) {
+                                                                int block_size, int max_blocks, int RV, int window,
+                                                                const float* __restrict__ sink) {
     typedef TileGeom<NB> G;
     __shared__ __attribute__((aligned(16))) unsigned char lds[G::LDS_BYTES];
     const int b = blockIdx.y;
@@ -34,7 +35,7 @@ __global__ __launch_bounds__(256) void latent_attn_tiles_kernel(const unsigned s
     latent_tile_loop<NB, NBV, 4>(q + ((size_t)q0 * H + rc) * R, cache, block_tables + (size_t)b * max_blocks, R, block_size, k_lo,
                                  k_hi, row_pos, wave_min_pos, c_log2, window, lds, oacc, m_run, l_tot);
     if (r >= rows) return;
-    const float inv = 1.f / l_tot;
+    const float inv = sink ? sink_inv(m_run * c_log2, l_tot, sink[r % H]) : 1.f / l_tot;
     unsigned short* op = o + ((size_t)q0 * H + r) * RV + 4 * hi;
 #pragma unroll
     for (int d = 0; d < NBV; ++d)
@@ -54,7 +55,7 @@ using namespace sm;
 
 extern "C" int sm_latent_attn_tiles(const void* q, const void* cache, const int32_t* block_tables, const int32_t* qstart,
                                     const int32_t* seq_pos0, void* o, float scale, int B, int max_q, int H, int R, int block_size,
-                                    int max_blocks, int RV, int window, void* stream) {
+                                    int max_blocks, int RV, int window, const float* sink, void* stream) {
     if (RV <= 0) RV = R;
     if (B < 0 || max_q < 0 || H < 1 || R < 1 || RV > R || window < 0 || block_size < 1 || max_blocks < 1 ||
         (B > 0 && max_q > 0 && (!q || !cache || !block_tables || !qstart || !seq_pos0 || !o))) {
@@ -74,7 +75,7 @@ extern "C" int sm_latent_attn_tiles(const void* q, const void* cache, const int3
 #define SM_TILES(NB_, NBV_)                                                                                               \
     hipLaunchKernelGGL((latent_attn_tiles_kernel<NB_, NBV_>), grid, block, 0, s, (const unsigned short*)q,                 \
                        (const unsigned short*)cache, block_tables, qstart, seq_pos0, (unsigned short*)o, c, H, R, block_size, \
-                       max_blocks, RV, window)
+                       max_blocks, RV, window, sink)
     SM_BY_LATENT_SIZE(nb, nbv, SM_TILES);
 #undef SM_TILES
     SM_CHECK_LAUNCH("sm_latent_attn_tiles");

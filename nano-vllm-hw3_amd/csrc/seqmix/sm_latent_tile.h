@@ -21,6 +21,13 @@ typedef short s16x8 __attribute__((ext_vector_type(8)));
 
 constexpr int kTileKeys = 64;
 
+// 1 / (softmax denominator) of a row whose scores reached m2 (log2 units) and summed to l relative to it, with one more term
+// exp(sink): relative to m2 again, so that the row's unnormalised output times this is its output
+__device__ __forceinline__ float sink_inv(float m2, float l, float sink) {
+    const float s2 = sink * 1.4426950408889634f, mx = fmaxf(m2, s2), f = __builtin_amdgcn_exp2f(m2 - mx);
+    return f / (l * f + __builtin_amdgcn_exp2f(s2 - mx));
+}
+
 template <int NB>
 struct TileGeom {
     static constexpr int RP = 32 * NB, CH = RP / 8, RS = RP * 2 + 16, LDS_BYTES = kTileKeys * RS;

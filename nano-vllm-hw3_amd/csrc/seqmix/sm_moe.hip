@@ -14,21 +14,24 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
                                                         int32_t* __restrict__ idx, float* __restrict__ wts, int64_t T_all, int W,
                                                         int E, int top, int groups, int keep, int score,
                                                         const float* __restrict__ correction, int group_top, int renorm,
-                                                        int staged, const float* __restrict__ bias) {
-    extern __shared__ float z_all[];             // per token: E scores, then `groups` group scores; then the staged rows
+                                                        int staged, const float* __restrict__ bias,
+                                                        const float* __restrict__ gate_w, float* __restrict__ gate_out) {
+    // per token: E scores, `groups` group scores and, with gate_w, the gate's logit; then the staged rows
+    extern __shared__ float z_all[];
+    const int RS = E + groups + (gate_w ? 1 : 0), rows = E + (gate_w ? 1 : 0);     // the gate's row follows the experts'
     const int64_t t0 = (int64_t)blockIdx.x * kRouteTokens;
     const int nt = (int)min((int64_t)kRouteTokens, T_all - t0);
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     if (staged) {
         // the workgroup's token rows (one contiguous piece of h) go to LDS once; every expert's row is then read once per
         // workgroup in 16-byte pieces and meets all the tokens there
-        T* h_lds = (T*)(z_all + kRouteTokens * (E + groups));
+        T* h_lds = (T*)(z_all + kRouteTokens * RS);
         const T* src = h + (size_t)t0 * W;
         struct alignas(sizeof(T) * 4) Pack4 { T v[4]; };
         for (int i = threadIdx.x * 4; i < nt * W; i += 1024) *(Pack4*)(h_lds + i) = *(const Pack4*)(src + i);     // W % 4 == 0
         __syncthreads();
-        for (int e = wave; e < E; e += 4) {
-            const float* wr = router_w + (size_t)e * W;
+        for (int e = wave; e < rows; e += 4) {
+            const float* wr = e < E ? router_w + (size_t)e * W : gate_w;
             float d[kRouteTokens];
             for (int i = 0; i < kRouteTokens; ++i) d[i] = 0.f;
             for (int c = lane * 4; c < W; c += 256) {
@@ -42,12 +45,12 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
             }
             for (int i = 0; i < kRouteTokens; ++i) {
                 const float sum = wave_sum(d[i]);
-                if (lane == 0) z_all[i * (E + groups) + e] = sum;
+                if (lane == 0) z_all[i * RS + (e < E ? e : RS - 1)] = sum;
             }
         }
     } else {
-        for (int e = wave; e < E; e += 4) {
-            const float* wr = router_w + (size_t)e * W;
+        for (int e = wave; e < rows; e += 4) {
+            const float* wr = e < E ? router_w + (size_t)e * W : gate_w;
             float d[kRouteTokens];
             for (int i = 0; i < kRouteTokens; ++i) d[i] = 0.f;
             for (int c = lane; c < W; c += 64) {
@@ -57,7 +60,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
             }
             for (int i = 0; i < kRouteTokens; ++i) {
                 const float sum = wave_sum(d[i]);
-                if (lane == 0) z_all[i * (E + groups) + e] = sum;
+                if (lane == 0) z_all[i * RS + (e < E ? e : RS - 1)] = sum;
             }
         }
     }
@@ -65,7 +68,8 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
     if (threadIdx.x >= nt) return;
     // one thread finishes a token: E is small and the selections are sequential by nature
     const int64_t t = t0 + threadIdx.x;
-    float* z = z_all + threadIdx.x * (E + groups);
+    float* z = z_all + threadIdx.x * RS;
+    if (gate_w != nullptr) gate_out[t] = 1.f / (1.f + expf(-z[RS - 1]));
     if (bias != nullptr)
         for (int e = 0; e < E; ++e) z[e] += bias[e];
     if (score == SM_ROUTE_SIGMOID) {
@@ -177,10 +181,12 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
 template <typename T>
 __global__ __launch_bounds__(256) void moe_pairs_gate_up_kernel(const T* __restrict__ h, const int32_t* __restrict__ idx,
                                                                 const T* __restrict__ w_gu, float limit, float alpha,
-                                                                T* __restrict__ act, int top, int W, int F, int act_kind) {
+                                                                T* __restrict__ act, int top, int W, int F, int act_kind,
+                                                                const float* __restrict__ in_wts) {
     extern __shared__ float h_lds[];
     const int64_t p = blockIdx.x, t = p / top;
     const int e = idx[p];
+    const float iw = in_wts ? in_wts[p] : 1.f;       // a weight on the expert's input: the products are linear in it
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     for (int c = threadIdx.x; c < W; c += 256) h_lds[c] = to_f(h[(size_t)t * W + c]);
     __syncthreads();
@@ -191,7 +197,7 @@ __global__ __launch_bounds__(256) void moe_pairs_gate_up_kernel(const T* __restr
             float u = 0.f;
             for (int c = lane; c < W; c += 64) u += h_lds[c] * to_f(u_row[c]);
             u = wave_sum(u);
-            if (lane == 0) act[(size_t)p * F + f] = from_f<T>(plain_act(to_f(from_f<T>(u)), act_kind));
+            if (lane == 0) act[(size_t)p * F + f] = from_f<T>(plain_act(to_f(from_f<T>(u * iw)), act_kind));
         }
         return;
     }
@@ -208,7 +214,7 @@ __global__ __launch_bounds__(256) void moe_pairs_gate_up_kernel(const T* __restr
         g = wave_sum(g);
         u = wave_sum(u);
         // the products leave the matrix unit in the storage type, as a GEMM's output would
-        if (lane == 0) act[(size_t)p * F + f] = from_f<T>(gated_act(to_f(from_f<T>(g)), to_f(from_f<T>(u)), limit, alpha, act_kind));
+        if (lane == 0) act[(size_t)p * F + f] = from_f<T>(gated_act(to_f(from_f<T>(g * iw)), to_f(from_f<T>(u * iw)), limit, alpha, act_kind));
     }
 }
 
@@ -217,7 +223,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void moe_pairs_down_kernel(const T* __restrict__ act, const int32_t* __restrict__ idx,
                                                              const float* __restrict__ wts, const T* __restrict__ w_down,
                                                              const T* __restrict__ shared, T* __restrict__ y, int top, int W, int F,
-                                                             int staged) {
+                                                             int staged, const float* __restrict__ shared_scale) {
     extern __shared__ float a_lds[];             // top * F activations of the token's pairs (staged: they fit)
     const int64_t t = blockIdx.x;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -238,10 +244,10 @@ __global__ __launch_bounds__(256) void moe_pairs_down_kernel(const T* __restrict
                 for (int c = lane; c < F; c += 64) d += to_f(a_row[k * F + c]) * to_f(row[c]);
             }
             d = wave_sum(d);
-            tot += wts[(size_t)t * top + k] * to_f(from_f<T>(d));
+            tot += (wts ? wts[(size_t)t * top + k] : 1.f) * to_f(from_f<T>(d));
         }
         if (lane == 0) {
-            if (shared) tot += to_f(shared[(size_t)t * W + w]);
+            if (shared) tot += (shared_scale ? shared_scale[t] : 1.f) * to_f(shared[(size_t)t * W + w]);
             y[(size_t)t * W + w] = from_f<T>(tot);
         }
     }
@@ -253,8 +259,8 @@ using namespace sm;
 
 extern "C" int sm_moe_route(int dtype, const void* h, const float* router_w, int32_t* idx, float* wts, int64_t T, int W, int E,
                             int top, int groups, int keep, int score, const float* correction, int group_top, int renorm,
-                            const float* bias, void* stream) {
-    if (T < 0 || W < 1 || E < 1 || top < 1 || (score != SM_ROUTE_SOFTMAX && score != SM_ROUTE_SIGMOID) || group_top < 1 ||
+                            const float* bias, const float* gate_w, float* gate_out, void* stream) {
+    if ((gate_w != nullptr) != (gate_out != nullptr) || T < 0 || W < 1 || E < 1 || top < 1 || (score != SM_ROUTE_SOFTMAX && score != SM_ROUTE_SIGMOID) || group_top < 1 ||
         group_top > 4 || (T > 0 && (!h || !router_w || !idx || !wts))) {
         set_error("sm_moe_route: bad argument");
         return SM_EINVAL;
@@ -266,20 +272,20 @@ extern "C" int sm_moe_route(int dtype, const void* h, const float* router_w, int
     }
     if (T == 0) return SM_OK;
     // the token rows of a workgroup are staged in LDS when they fit and the rows can be moved in pieces of four channels
-    const size_t scores = (size_t)kRouteTokens * (E + groups) * 4;
+    const size_t scores = (size_t)kRouteTokens * (E + groups + (gate_w ? 1 : 0)) * 4;
     const size_t rows = (size_t)kRouteTokens * W * (dtype == SM_F32 ? 4 : 2);
-    const int staged = W % 4 == 0 && scores % 16 == 0 && scores + rows <= 60 * 1024 && ((uintptr_t)h | (uintptr_t)router_w) % 16 == 0;
+    const int staged = W % 4 == 0 && scores % 16 == 0 && scores + rows <= 60 * 1024 && ((uintptr_t)h | (uintptr_t)router_w | (uintptr_t)gate_w) % 16 == 0;
     SM_DISPATCH(dtype, "sm_moe_route",
                 hipLaunchKernelGGL(moe_route_kernel<DT>, dim3((unsigned)((T + kRouteTokens - 1) / kRouteTokens)), dim3(256),
                                    scores + (staged ? rows : 0), as_stream(stream), (const DT*)h, router_w, idx, wts, T, W, E,
-                                   top, groups, keep, score, correction, group_top, renorm, staged, bias));
+                                   top, groups, keep, score, correction, group_top, renorm, staged, bias, gate_w, gate_out));
     SM_CHECK_LAUNCH("sm_moe_route");
     return SM_OK;
 }
 
 extern "C" int sm_moe_pairs_gate_up(int dtype, const void* h, const int32_t* idx, const void* w_gu, float limit, float alpha,
-                                    int act_kind, void* act, int64_t T, int top, int W, int F, void* stream) {
-    if (T < 0 || top < 1 || W < 1 || F < 1 || act_kind < 0 || act_kind > SM_ACT_SILU_GLU || (T > 0 && (!h || !idx || !w_gu || !act))) {
+                                    int act_kind, const float* in_wts, void* act, int64_t T, int top, int W, int F, void* stream) {
+    if (T < 0 || top < 1 || W < 1 || F < 1 || act_kind < 0 || act_kind > SM_ACT_LAST || (T > 0 && (!h || !idx || !w_gu || !act))) {
         set_error("sm_moe_pairs_gate_up: bad argument");
         return SM_EINVAL;
     }
@@ -287,14 +293,16 @@ extern "C" int sm_moe_pairs_gate_up(int dtype, const void* h, const int32_t* idx
     if (T == 0) return SM_OK;
     SM_DISPATCH(dtype, "sm_moe_pairs_gate_up",
                 hipLaunchKernelGGL(moe_pairs_gate_up_kernel<DT>, dim3((unsigned)(T * top)), dim3(256), (size_t)W * 4,
-                                   as_stream(stream), (const DT*)h, idx, (const DT*)w_gu, limit, alpha, (DT*)act, top, W, F, act_kind));
+                                   as_stream(stream), (const DT*)h, idx, (const DT*)w_gu, limit, alpha, (DT*)act, top, W, F, act_kind,
+                                   in_wts));
     SM_CHECK_LAUNCH("sm_moe_pairs_gate_up");
     return SM_OK;
 }
 
 extern "C" int sm_moe_pairs_down(int dtype, const void* act, const int32_t* idx, const float* wts, const void* w_down,
-                                 const void* shared, void* y, int64_t T, int top, int W, int F, void* stream) {
-    if (T < 0 || top < 1 || W < 1 || F < 1 || (T > 0 && (!act || !idx || !wts || !w_down || !y))) {
+                                 const void* shared, const float* shared_scale, void* y, int64_t T, int top, int W, int F,
+                                 void* stream) {
+    if (T < 0 || top < 1 || W < 1 || F < 1 || (shared_scale && !shared) || (T > 0 && (!act || !idx || !w_down || !y))) {
         set_error("sm_moe_pairs_down: bad argument");
         return SM_EINVAL;
     }
@@ -303,7 +311,7 @@ extern "C" int sm_moe_pairs_down(int dtype, const void* act, const int32_t* idx,
     SM_DISPATCH(dtype, "sm_moe_pairs_down",
                 hipLaunchKernelGGL(moe_pairs_down_kernel<DT>, dim3((unsigned)T), dim3(256), staged ? (size_t)top * F * 4 : 0,
                                    as_stream(stream), (const DT*)act, idx, wts, (const DT*)w_down, (const DT*)shared, (DT*)y, top, W,
-                                   F, staged));
+                                   F, staged, shared_scale));
     SM_CHECK_LAUNCH("sm_moe_pairs_down");
     return SM_OK;
 }

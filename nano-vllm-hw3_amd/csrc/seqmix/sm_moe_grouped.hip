@@ -59,12 +59,13 @@ __device__ __forceinline__ bf16x8 load8(const unsigned short* p, int k, int K) {
 
 // GATE_UP: A = h rows gathered by token, B = the expert's gate and up rows, out = act [rows, N] (N = F, K = W)
 // else:    A = act rows,                 B = the expert's down rows,       out = per-row products [rows, N] (N = W, K = F)
-// MODE 0: the down product; 1: gate and up with the gated activation (act_kind: clamped GLU or silu(g) u); 2: the up product alone with a GELU (act_kind)
+// MODE 0: the down product; 1: gate and up with a gated activation (act_kind); 2: the up product alone with a plain one.
+// in_wts != NULL (modes 1, 2): pair p's products are scaled by in_wts[p] before the activation (a weight on the expert's input)
 template <int MODE>
 __global__ __launch_bounds__(256) void moe_grouped_kernel(const unsigned short* __restrict__ a, const unsigned short* __restrict__ w,
                                                           const int32_t* __restrict__ row_pair, const int32_t* __restrict__ tile_expert,
                                                           unsigned short* __restrict__ out, int top, int N, int K, float limit,
-                                                          float alpha, int act_kind) {
+                                                          float alpha, int act_kind, const float* __restrict__ in_wts) {
     constexpr bool GATE_UP = MODE == 1, FROM_TOKENS = MODE != 0;
     const int tile = blockIdx.x;
     const int e = tile_expert[tile];
@@ -120,23 +121,26 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(const unsigned short* 
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
         const int orow = tile * kRowsPerTile + (r & 3) + 8 * (r >> 2) + 4 * hi;
-        if (row_pair[orow] < 0) continue;
-        const float v = GATE_UP ? glu_bf16(acc[r], acc2[r], limit, alpha, act_kind) : (MODE == 2 ? plain_act((float)(bf16_t)acc[r], act_kind) : acc[r]);
+        const int p = row_pair[orow];
+        if (p < 0) continue;
+        const float iw = FROM_TOKENS && in_wts ? in_wts[p] : 1.f;
+        const float v = GATE_UP ? glu_bf16(acc[r] * iw, acc2[r] * iw, limit, alpha, act_kind)
+                                : (MODE == 2 ? plain_act((float)(bf16_t)(acc[r] * iw), act_kind) : acc[r]);
         out[(size_t)orow * N + n0 + l31] = __builtin_bit_cast(unsigned short, (bf16_t)v);
     }
 }
 
 __global__ void moe_combine_kernel(const unsigned short* __restrict__ prod, const int32_t* __restrict__ pair_row,
                                    const float* __restrict__ wts, const unsigned short* __restrict__ shared,
-                                   unsigned short* __restrict__ y, int top, int W) {
+                                   unsigned short* __restrict__ y, int top, int W, const float* __restrict__ shared_scale) {
     const size_t t = blockIdx.x;
     for (int c = threadIdx.x; c < W; c += blockDim.x) {
         float tot = 0.f;
         for (int k = 0; k < top; ++k) {
             const size_t r = pair_row[t * top + k];
-            tot += wts[t * top + k] * (float)__builtin_bit_cast(bf16_t, prod[r * W + c]);
+            tot += (wts ? wts[t * top + k] : 1.f) * (float)__builtin_bit_cast(bf16_t, prod[r * W + c]);
         }
-        if (shared) tot += (float)__builtin_bit_cast(bf16_t, shared[t * W + c]);
+        if (shared) tot += (shared_scale ? shared_scale[t] : 1.f) * (float)__builtin_bit_cast(bf16_t, shared[t * W + c]);
         y[t * W + c] = __builtin_bit_cast(unsigned short, (bf16_t)tot);
     }
 }
@@ -151,10 +155,10 @@ extern "C" int sm_moe_grouped_tiles(int64_t T, int top, int E) {
 }
 
 extern "C" int sm_moe_grouped(const void* h, const int32_t* idx, const float* wts, const void* w_gu, const void* w_down,
-                              const void* shared, float limit, float alpha, int act_kind, void* y, int64_t T, int top, int E, int W, int F,
+                              const void* shared, const float* shared_scale, int weight_in, float limit, float alpha, int act_kind, void* y, int64_t T, int top, int E, int W, int F,
                               int32_t* row_pair, int32_t* tile_expert, int32_t* pair_row, void* act, void* prod, void* stream) {
-    if (T < 0 || top < 1 || E < 1 || W < 1 || F < 1 || act_kind < 0 || act_kind > SM_ACT_SILU_GLU ||
-        (T > 0 && (!h || !idx || !wts || !w_gu || !w_down || !y || !row_pair || !tile_expert || !pair_row || !act || !prod))) {
+    if (T < 0 || top < 1 || E < 1 || W < 1 || F < 1 || act_kind < 0 || act_kind > SM_ACT_LAST ||
+        (T > 0 && (!h || !idx || !wts || !w_gu || !w_down || !row_pair || !tile_expert || !pair_row || !act || !prod))) {
         set_error("sm_moe_grouped: bad argument");
         return SM_EINVAL;
     }
@@ -168,23 +172,21 @@ extern "C" int sm_moe_grouped(const void* h, const int32_t* idx, const float* wt
     hipLaunchKernelGGL(moe_align_kernel, dim3(1), dim3(1024), (size_t)3 * E * sizeof(int), s, idx, (int)(T * top), E, tiles, row_pair,
                        tile_expert, pair_row);
     SM_CHECK_LAUNCH("sm_moe_grouped (align)");
-    if (act_kind == SM_ACT_CLAMPED_GLU || act_kind == SM_ACT_SILU_GLU)
+    if (act_is_gated(act_kind))
         hipLaunchKernelGGL(moe_grouped_kernel<1>, dim3((unsigned)tiles, (unsigned)((F + 127) / 128)), dim3(256), 0, s,
                            (const unsigned short*)h, (const unsigned short*)w_gu, row_pair, tile_expert, (unsigned short*)act, top, F,
-                           W, limit, alpha, act_kind);
+                           W, limit, alpha, act_kind, weight_in ? wts : nullptr);
     else
         hipLaunchKernelGGL(moe_grouped_kernel<2>, dim3((unsigned)tiles, (unsigned)((F + 127) / 128)), dim3(256), 0, s,
                            (const unsigned short*)h, (const unsigned short*)w_gu, row_pair, tile_expert, (unsigned short*)act, top, F,
-                           W, limit, alpha, act_kind);
+                           W, limit, alpha, act_kind, weight_in ? wts : nullptr);
     SM_CHECK_LAUNCH("sm_moe_grouped (gate/up)");
     hipLaunchKernelGGL(moe_grouped_kernel<0>, dim3((unsigned)tiles, (unsigned)((W + 127) / 128)), dim3(256), 0, s,
                        (const unsigned short*)act, (const unsigned short*)w_down, row_pair, tile_expert, (unsigned short*)prod, top, W,
-                       F, 0.f, 0.f, 0);
+                       F, 0.f, 0.f, 0, (const float*)nullptr);
     SM_CHECK_LAUNCH("sm_moe_grouped (down)");
-    hipLaunchKernelGGL(moe_combine_kernel, dim3((unsigned)T), dim3(256), 0, s, (const unsigned short*)prod, pair_row, wts,
-                       (const unsigned short*)shared, (unsigned short*)y, top, W);
-    SM_CHECK_LAUNCH("sm_moe_grouped (combine)");
-    return SM_OK;
+    if (y == nullptr) return SM_OK;               // the caller sums a token's pairs itself
+    return sm_moe_combine(prod, pair_row, weight_in ? nullptr : wts, shared, shared_scale, y, T, top, W, stream);
 }
 
 // The grouping and the final sum on their own, for callers that run the expert products themselves (the engine gives
@@ -202,15 +204,15 @@ extern "C" int sm_moe_align(const int32_t* idx, int64_t T, int top, int E, int32
     return SM_OK;
 }
 
-extern "C" int sm_moe_combine(const void* prod, const int32_t* pair_row, const float* wts, const void* shared, void* y, int64_t T,
-                              int top, int W, void* stream) {
-    if (T < 0 || top < 1 || W < 1 || (T > 0 && (!prod || !pair_row || !wts || !y))) {
+extern "C" int sm_moe_combine(const void* prod, const int32_t* pair_row, const float* wts, const void* shared,
+                              const float* shared_scale, void* y, int64_t T, int top, int W, void* stream) {
+    if (T < 0 || top < 1 || W < 1 || (shared_scale && !shared) || (T > 0 && (!prod || !pair_row || !y))) {
         set_error("sm_moe_combine: bad argument");
         return SM_EINVAL;
     }
     if (T == 0) return SM_OK;
     hipLaunchKernelGGL(moe_combine_kernel, dim3((unsigned)T), dim3(256), 0, as_stream(stream), (const unsigned short*)prod, pair_row,
-                       wts, (const unsigned short*)shared, (unsigned short*)y, top, W);
+                       wts, (const unsigned short*)shared, (unsigned short*)y, top, W, shared_scale);
     SM_CHECK_LAUNCH("sm_moe_combine");
     return SM_OK;
 }

@@ -62,12 +62,13 @@ __device__ __forceinline__ i32x4 load16(const unsigned short* p, int k, int K) {
 
 // GATE_UP: A = h rows gathered by token, B = the expert's gate and up rows, out = act [rows, N] (N = F, K = W)
 // else:    A = act rows,                 B = the expert's down rows,       out = per-row products [rows, N] (N = W, K = F)
-// MODE 0: the down product; 1: gate and up with the gated activation (act_kind: clamped GLU or silu(g) u); 2: the up product alone with a GELU (act_kind)
+// MODE 0: the down product; 1: gate and up with a gated activation (act_kind); 2: the up product alone with a plain one.
+// in_wts != NULL (modes 1, 2): pair p's products are scaled by in_wts[p] before the activation (a weight on the expert's input)
 template <int MODE>
 __global__ __launch_bounds__(256) void moe_tiles128_kernel(const unsigned short* __restrict__ a, const unsigned short* __restrict__ w,
                                                            const int32_t* __restrict__ row_pair, const int32_t* __restrict__ tile_expert,
                                                            unsigned short* __restrict__ out, int top, int N, int K, float limit,
-                                                           float alpha, int act_kind) {
+                                                           float alpha, int act_kind, const float* __restrict__ in_wts) {
     __shared__ __attribute__((aligned(16))) unsigned char a_lds[kBigRows * kAStride];
     constexpr bool GATE_UP = MODE == 1, FROM_TOKENS = MODE != 0;
     const int tile = blockIdx.x;
@@ -130,9 +131,11 @@ __global__ __launch_bounds__(256) void moe_tiles128_kernel(const unsigned short*
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
             const int orow = tile * kBigRows + 32 * m + (r & 3) + 8 * (r >> 2) + 4 * hi;
-            if (row_pair[orow] < 0) continue;
-            const float v = GATE_UP ? glu_bf16_big(acc[m][r], acc2[m][r], limit, alpha, act_kind)
-                                    : (MODE == 2 ? plain_act((float)(bf16_t)acc[m][r], act_kind) : acc[m][r]);
+            const int p = row_pair[orow];
+            if (p < 0) continue;
+            const float iw = FROM_TOKENS && in_wts ? in_wts[p] : 1.f;
+            const float v = GATE_UP ? glu_bf16_big(acc[m][r] * iw, acc2[m][r] * iw, limit, alpha, act_kind)
+                                    : (MODE == 2 ? plain_act((float)(bf16_t)(acc[m][r] * iw), act_kind) : acc[m][r]);
             out[(size_t)orow * N + n0 + l31] = __builtin_bit_cast(unsigned short, (bf16_t)v);
         }
 }
@@ -147,10 +150,10 @@ extern "C" int sm_moe_tiles128_count(int64_t T, int top, int E) {
 }
 
 extern "C" int sm_moe_tiles128(const void* h, const int32_t* idx, const float* wts, const void* w_gu, const void* w_down,
-                               const void* shared, float limit, float alpha, int act_kind, void* y, int64_t T, int top, int E, int W, int F,
+                               const void* shared, const float* shared_scale, int weight_in, float limit, float alpha, int act_kind, void* y, int64_t T, int top, int E, int W, int F,
                                int32_t* row_pair, int32_t* tile_expert, int32_t* pair_row, void* act, void* prod, void* stream) {
-    if (T < 0 || top < 1 || E < 1 || W < 1 || F < 1 || act_kind < 0 || act_kind > SM_ACT_SILU_GLU ||
-        (T > 0 && (!h || !idx || !wts || !w_gu || !w_down || !y || !row_pair || !tile_expert || !pair_row || !act || !prod))) {
+    if (T < 0 || top < 1 || E < 1 || W < 1 || F < 1 || act_kind < 0 || act_kind > SM_ACT_LAST ||
+        (T > 0 && (!h || !idx || !wts || !w_gu || !w_down || !row_pair || !tile_expert || !pair_row || !act || !prod))) {
         set_error("sm_moe_tiles128: bad argument");
         return SM_EINVAL;
     }
@@ -164,18 +167,19 @@ extern "C" int sm_moe_tiles128(const void* h, const int32_t* idx, const float* w
     hipLaunchKernelGGL(moe_align128_kernel, dim3(1), dim3(1024), (size_t)3 * E * sizeof(int), s, idx, (int)(T * top), E, tiles, row_pair,
                        tile_expert, pair_row);
     SM_CHECK_LAUNCH("sm_moe_tiles128 (align)");
-    if (act_kind == SM_ACT_CLAMPED_GLU || act_kind == SM_ACT_SILU_GLU)
+    if (act_is_gated(act_kind))
         hipLaunchKernelGGL(moe_tiles128_kernel<1>, dim3((unsigned)tiles, (unsigned)((F + 127) / 128)), dim3(256), 0, s,
                            (const unsigned short*)h, (const unsigned short*)w_gu, row_pair, tile_expert, (unsigned short*)act, top, F,
-                           W, limit, alpha, act_kind);
+                           W, limit, alpha, act_kind, weight_in ? wts : nullptr);
     else
         hipLaunchKernelGGL(moe_tiles128_kernel<2>, dim3((unsigned)tiles, (unsigned)((F + 127) / 128)), dim3(256), 0, s,
                            (const unsigned short*)h, (const unsigned short*)w_gu, row_pair, tile_expert, (unsigned short*)act, top, F,
-                           W, limit, alpha, act_kind);
+                           W, limit, alpha, act_kind, weight_in ? wts : nullptr);
     SM_CHECK_LAUNCH("sm_moe_tiles128 (gate/up)");
     hipLaunchKernelGGL(moe_tiles128_kernel<0>, dim3((unsigned)tiles, (unsigned)((W + 127) / 128)), dim3(256), 0, s,
                        (const unsigned short*)act, (const unsigned short*)w_down, row_pair, tile_expert, (unsigned short*)prod, top, W,
-                       F, 0.f, 0.f, 0);
+                       F, 0.f, 0.f, 0, (const float*)nullptr);
     SM_CHECK_LAUNCH("sm_moe_tiles128 (down)");
-    return sm_moe_combine(prod, pair_row, wts, shared, y, T, top, W, stream);
+    if (y == nullptr) return SM_OK;               // the caller sums a token's pairs itself
+    return sm_moe_combine(prod, pair_row, weight_in ? nullptr : wts, shared, shared_scale, y, T, top, W, stream);
 }

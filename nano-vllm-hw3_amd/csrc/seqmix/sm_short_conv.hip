@@ -1,0 +1,117 @@
+// Short causal convolution over time on every channel, with the last taps-1 inputs of every sequence carried as state
+// between steps; optionally with a bias, a SiLU behind it, or the input added to the result.  One launch convolves and
+// moves the state: a thread owns VEC channels and walks kChunk tokens of one sequence's portion with the last taps-1 inputs
+// in registers; only a portion's first chunk reads the carried inputs (kChunk >= taps-1), and the same threads write the
+// new ones afterwards, so no other workgroup reads what they change.
+#include "sm_common.h"
+
+namespace sm {
+
+constexpr int kMaxTaps = 16, kChunk = 16;
+
+// TAPS = the register form's size; taps <= TAPS are the convolution's (the first TAPS - taps columns do not exist)
+template <typename T, int VEC, int TAPS>
+__global__ __launch_bounds__(64) void short_conv_kernel(const T* __restrict__ x, int64_t row_stride, const T* __restrict__ w,
+                                                        const T* __restrict__ bias, int silu, int add_input, T* state, int run,
+                                                        int runs, const int32_t* __restrict__ qstart,
+                                                        const int32_t* __restrict__ seq_pos0, const int32_t* __restrict__ seq_slot,
+                                                        T* __restrict__ out, int W, int taps) {
+    struct alignas(sizeof(T) * VEC) Pack { T v[VEC]; };
+    const int b = blockIdx.z;
+    const int q0 = qstart[b], n = qstart[b + 1] - q0, t0 = blockIdx.x * kChunk;
+    const int c = (blockIdx.y * 64 + threadIdx.x) * VEC;
+    if (t0 >= n || c >= W) return;
+    const int pos0 = seq_pos0[b], skip = TAPS - taps;
+    T* st = state + ((size_t)seq_slot[b] * runs + run) * (size_t)(taps - 1) * W + c;      // (taps == 1: not touched)
+    const T* xc = x + (size_t)q0 * row_stride + c;
+    float wr[TAPS][VEC], hist[TAPS][VEC], bs[VEC];
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) wr[j][e] = j >= skip ? to_f(w[(size_t)(c + e) * taps + j - skip]) : 0.f;
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) bs[e] = bias ? to_f(bias[c + e]) : 0.f;
+    // hist[j] = the input TAPS - 1 - j tokens before the current one: rows of this step, then the carried inputs (state row
+    // k = the input taps-1-k tokens before the portion), zero before the sequence's start whatever the slot holds
+#pragma unroll
+    for (int j = 0; j < TAPS - 1; ++j) {
+        const int idx = t0 - (TAPS - 1) + j;
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) hist[j][e] = 0.f;
+        if (j < skip || pos0 + idx < 0) continue;
+        const Pack v = idx >= 0 ? *(const Pack*)(xc + (size_t)idx * row_stride) : *(const Pack*)(st + (size_t)(idx + taps - 1) * W);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) hist[j][e] = to_f(v.v[e]);
+    }
+    const int nt = min(kChunk, n - t0);
+    auto step = [&](int i) {
+        const Pack cur = *(const Pack*)(xc + (size_t)(t0 + i) * row_stride);
+        Pack o;
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) {
+            const float v = to_f(cur.v[e]);
+            float acc = bs[e] + wr[TAPS - 1][e] * v;
+#pragma unroll
+            for (int j = 0; j < TAPS - 1; ++j) acc += wr[j][e] * hist[j][e];
+            if (silu) acc = acc / (1.f + __expf(-acc));
+            o.v[e] = from_f<T>(add_input ? v + acc : acc);
+#pragma unroll
+            for (int j = 0; j + 1 < TAPS - 1; ++j) hist[j][e] = hist[j + 1][e];
+            if (TAPS > 1) hist[TAPS > 1 ? TAPS - 2 : 0][e] = v;
+        }
+        *(Pack*)(out + (size_t)(q0 + t0 + i) * W + c) = o;
+    };
+    if (nt == kChunk) {
+#pragma unroll 4
+        for (int i = 0; i < kChunk; ++i) step(i);
+    } else {
+        for (int i = 0; i < nt; ++i) step(i);
+    }
+    if (blockIdx.x != 0 || taps == 1) return;
+    for (int k = 0; k < taps - 1; ++k) {           // ascending: a row is read (k + n > k) before it is replaced
+        const int src = n - (taps - 1) + k;        // index inside the portion of the input that lands at k
+        *(Pack*)(st + (size_t)k * W) = src >= 0 ? *(const Pack*)(xc + (size_t)src * row_stride) : *(const Pack*)(st + (size_t)(k + n) * W);
+    }
+}
+
+template <typename T, int VEC>
+static void launch_short_conv(dim3 grid, hipStream_t s, const void* x, int64_t row_stride, const void* w, const void* bias, int silu,
+                              int add_input, void* state, int run, int runs, const int32_t* qstart, const int32_t* seq_pos0,
+                              const int32_t* seq_slot, void* out, int W, int taps) {
+#define SM_CONV(VEC_, TAPS_)                                                                                                     \
+    hipLaunchKernelGGL((short_conv_kernel<T, VEC_, TAPS_>), grid, dim3(64), 0, s, (const T*)x, row_stride, (const T*)w, (const T*)bias, \
+                       silu, add_input, (T*)state, run, runs, qstart, seq_pos0, seq_slot, (T*)out, W, taps)
+    if (taps <= 4) { SM_CONV(VEC, 4); return; }
+    grid.y = (unsigned)((W + 63) / 64);            // many taps: one channel per thread keeps the inputs in registers
+    SM_CONV(1, kMaxTaps);
+#undef SM_CONV
+}
+
+}  // namespace sm
+
+using namespace sm;
+
+extern "C" int sm_short_conv(int dtype, const void* x, int64_t row_stride, const void* w, const void* bias, int silu, int add_input,
+                             void* state, int run, int runs, const int32_t* qstart, const int32_t* seq_pos0,
+                             const int32_t* seq_slot, void* out, int B, int max_q, int W, int taps, void* stream) {
+    if (B < 0 || max_q < 0 || W < 1 || taps < 1 || run < 0 || run >= runs || row_stride < W ||
+        (B > 0 && max_q > 0 && (!x || !w || !qstart || !seq_pos0 || !seq_slot || !out || (taps > 1 && !state)))) {
+        set_error("sm_short_conv: bad argument");
+        return SM_EINVAL;
+    }
+    if (taps > kMaxTaps || B > 65535 || W > 64 * 65535) {
+        set_error("sm_short_conv: at most %d taps, 65535 sequences", kMaxTaps);
+        return SM_ESHAPE;
+    }
+    if (B == 0 || max_q == 0) return SM_OK;
+    const int full = dtype == SM_BF16 ? 8 : 4;     // 16-byte packs where every row and the state rows start on one
+    const bool wide = W % full == 0 && row_stride % full == 0 && ((uintptr_t)x | (uintptr_t)state | (uintptr_t)out) % 16 == 0;
+    const int vec = wide ? full : 1;
+    const dim3 grid((unsigned)((max_q + kChunk - 1) / kChunk), (unsigned)((W + 64 * vec - 1) / (64 * vec)), (unsigned)B);
+#define SM_CONV_ARGS grid, as_stream(stream), x, row_stride, w, bias, silu, add_input, state, run, runs, qstart, seq_pos0, seq_slot, out, W, taps
+    SM_DISPATCH(dtype, "sm_short_conv",
+                if (wide) launch_short_conv<DT, sizeof(DT) == 2 ? 8 : 4>(SM_CONV_ARGS); else launch_short_conv<DT, 1>(SM_CONV_ARGS));
+#undef SM_CONV_ARGS
+    SM_CHECK_LAUNCH("sm_short_conv");
+    return SM_OK;
+}

@@ -1,7 +1,7 @@
 """ctypes binding of libhymix.so (the C ABI declared in include/hymix.h): scaled embedding, the gated sublayer boundary
 with norms on both sides, token shift with carried state, rotary attention over a paged key/value cache with sinks and
 windows, chunked masks and sigmoid weights, the generalized delta rule and linear attention with a constant decay with their
-per-sequence states, squared ReLU, the grouped-norm and tanh-norm residual boundaries.  No fallback on a GPU: a missing library
+per-sequence states, the selective scan, squared ReLU, the grouped-norm, tanh-norm and layer-norm residual boundaries.  No fallback on a GPU: a missing library
 raises (``build_if_missing`` compiles it in-tree first, which needs hipcc but no GPU)."""
 import ctypes
 import os
@@ -38,11 +38,14 @@ SIGNATURES = {
                                        _int, _vp]),
     "hm_dyt_residual": (_int, [_int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _int, _vp]),
     "hm_group_norm_residual": (_int, [_int, _vp, _vp, _vp, _vp, _vp, _int, _f, _vp, _i64, _int, _vp]),
+    "hm_layer_norm_residual": (_int, [_int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _int, _vp, _f, _vp, _i64, _int, _vp]),
+    "hm_selective_scan": (_int, [_int, _vp, _i64, _vp, _i64, _vp, _vp, _i64, _int, _int, _vp, _vp, _vp, _i64, _vp, _vp, _vp, _vp, _vp,
+                                 _i64, _int, _int, _int, _int, _vp]),
     "hm_scale_softcap": (_int, [_vp, _i64, _f, _f, _vp]),
     "hm_delta_prepare": (_int, [_int, _vp, _i64, _int, _int, _int, _int, _vp, _vp, _vp, _int, _f, _f, _vp, _i64, _int, _int, _vp]),
     "hm_delta_recurrence": (_int, [_int, _vp, _vp, _i64, _vp, _vp, _vp, _vp, _vp, _int, _int, _int, _int, _vp]),
     "hm_delta_gate_norm": (_int, [_int, _vp, _vp, _i64, _vp, _f, _vp, _i64, _int, _int, _vp]),
-    "hm_relu_squared": (_int, [_int, _vp, _i64, _vp, _i64, _int, _vp]),
+    "hm_relu_squared": (_int, [_int, _vp, _i64, _vp, _vp, _i64, _i64, _int, _vp]),
 }
 
 _lib = None

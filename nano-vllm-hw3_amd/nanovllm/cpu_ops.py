@@ -101,7 +101,7 @@ def stream_step(X, y, mix, out, w_in, norm_w, eps, dtype):
     return (u * torch.rsqrt(u.pow(2).mean(-1, keepdim=True) + eps) * norm_w.float()).to(dtype)
 
 
-def canon_conv(h, w, state, run, ctx):
+def short_conv(h, w, state, run, ctx, bias=None, silu=False, add_input=False):
     taps = w.shape[1]
     out = torch.empty_like(h)
     qs = ctx.qstart.tolist()
@@ -110,15 +110,17 @@ def canon_conv(h, w, state, run, ctx):
         if e <= a:
             continue
         slot, pos0 = int(ctx.seq_slot[b]), int(ctx.seq_pos0[b])
-        prev = state[slot, run][:taps - 1].float().clone()                     # [taps-1, W]: inputs at pos0-(taps-1) .. pos0-1
+        # [taps-1, W]: inputs at pos0-(taps-1) .. pos0-1
+        prev = state[slot, run][:taps - 1].float().clone() if taps > 1 else h[:0].float()
         for k in range(taps - 1):
             if pos0 - (taps - 1) + k < 0:
                 prev[k] = 0
         hist = torch.cat([prev, h[a:e].float()], 0)
-        acc = h[a:e].float().clone()
+        acc = torch.zeros_like(h[a:e], dtype=torch.float32) if bias is None else bias.float().expand(e - a, -1).clone()
         for j in range(taps):
             acc += w[:, j].float() * hist[j:j + e - a]
-        out[a:e] = acc.to(h.dtype)
+        acc = F.silu(acc) if silu else acc
+        out[a:e] = (acc + h[a:e].float() if add_input else acc).to(h.dtype)
         if taps > 1:
             state[slot, run] = hist[-(taps - 1):].to(state.dtype)
     return out
@@ -131,13 +133,14 @@ def latent_norm_store(x, w, eps, cache, slot_mapping):
     cache.view(-1, cache.shape[-1])[slot_mapping[keep].long()] = c[keep]
 
 
-def rotate_pairs(x, pos, inv_freq, rot_dims):
-    """Channels (2i, 2i + 1), i < rot_dims / 2, of the last dimension turned by pos * inv_freq[i]; x [T, ..., C] f32."""
+def rotate_pairs(x, pos, inv_freq, rot_dims, mag=1.0):
+    """Channels (2i, 2i + 1), i < rot_dims / 2, of the last dimension turned by pos * inv_freq[i] (cosines and sines times
+    ``mag``); x [T, ..., C] f32."""
     if not rot_dims:
         return x
     ang = pos.float()[:, None] * inv_freq.float()[None, :]
     shape = [x.shape[0]] + [1] * (x.dim() - 2) + [rot_dims // 2]
-    c, s = torch.cos(ang).view(shape), torch.sin(ang).view(shape)
+    c, s = torch.cos(ang).view(shape) * mag, torch.sin(ang).view(shape) * mag
     u, v = x[..., 0:rot_dims:2], x[..., 1:rot_dims:2]
     out = x.clone()
     out[..., 0:rot_dims:2] = u * c - v * s
@@ -150,19 +153,20 @@ def rms_norm_rows(x, w, eps):
     return (xf * torch.rsqrt(xf.pow(2).mean(-1, keepdim=True) + eps) * w.float()).to(x.dtype)
 
 
-def latent_rope_store(x, w, eps, q, qa, inv_freq, rot_dims, H, D, R, Rd, cache, ctx):
-    T = x.shape[0]
-    xf = x.float()
-    c = xf[:, :R] * torch.rsqrt(xf[:, :R].pow(2).mean(-1, keepdim=True) + eps) * w.float()
-    kr = rotate_pairs(xf[:, R:], ctx.tok_pos, inv_freq, rot_dims)
-    rows = ctx.slot_mapping
-    keep = rows >= 0
-    cache.view(-1, R + Rd)[rows[keep].long()] = torch.cat([c, kr], -1).to(cache.dtype)[keep]
-    qr = rotate_pairs(q.float().view(T, H, D + Rd)[..., D:], ctx.tok_pos, inv_freq, rot_dims)
+def latent_rope_store(x, w, eps, q, qa, inv_freq, rot_dims, H, D, R, Rd, cache, ctx, mag=1.0):
+    T = q.shape[0]
+    if x is not None:
+        xf = x.float()
+        c = xf[:, :R] * torch.rsqrt(xf[:, :R].pow(2).mean(-1, keepdim=True) + eps) * w.float()
+        kr = rotate_pairs(xf[:, R:], ctx.tok_pos, inv_freq, rot_dims, mag)
+        rows = ctx.slot_mapping
+        keep = rows >= 0
+        cache.view(-1, R + Rd)[rows[keep].long()] = torch.cat([c, kr], -1).to(cache.dtype)[keep]
+    qr = rotate_pairs(q.float().view(T, H, D + Rd)[..., D:], ctx.tok_pos, inv_freq, rot_dims, mag)
     qa[..., R:] = qr.to(qa.dtype)
 
 
-def latent_attention(q, cache, ctx, scale, RV=0, window=0):
+def latent_attention(q, cache, ctx, scale, RV=0, window=0, sink=None):
     RV = RV or q.shape[-1]
     o = torch.empty(q.shape[:-1] + (RV,), dtype=q.dtype)
     bs = cache.shape[1]
@@ -181,7 +185,9 @@ def latent_attention(q, cache, ctx, scale, RV=0, window=0):
         if window > 0:
             hidden = hidden | (pos[:, None, None] - t[None, None, :] >= window)
         s = s.masked_fill(hidden, float("-inf"))
-        o[a:e] = torch.einsum("thn,nr->thr", torch.softmax(s, -1), c[:, :RV]).to(q.dtype)
+        if sink is not None:
+            s = torch.cat([s, sink.float()[None, :, None].expand(e - a, -1, 1)], -1)
+        o[a:e] = torch.einsum("thn,nr->thr", torch.softmax(s, -1)[..., :n], c[:, :RV]).to(q.dtype)
     return o
 
 
@@ -219,21 +225,33 @@ def moe_route(h, router_w, top, groups, keep, score=0, correction=None, group_to
     return idx.int(), (w / (w.sum(-1, keepdim=True) + 1e-20) if renorm else w)
 
 
-def moe_experts(h, idx, wts, w_gu, w_down, limit, alpha, shared, act_kind=0):
+def expert_act(z, act_kind, limit, alpha):
+    """The activation between a feed-forward's two products (seq_ops.ACT_*); z [T, 2F] = gate | up for the gated forms."""
+    if act_kind == 0:
+        return clamped_glu(z, limit, alpha)
+    if act_kind == 3:
+        g, u = z.float().chunk(2, -1)
+        g, u = g.clamp(max=limit), u.clamp(-limit, limit)
+        return (g * torch.sigmoid(alpha * g) * u).to(z.dtype)
+    if act_kind == 4:
+        return torch.relu(z.float()).pow(2).to(z.dtype)
+    if act_kind == 5:
+        g, u = z.float().chunk(2, -1)
+        return (F.gelu(g, approximate="tanh") * u).to(z.dtype)
+    return F.gelu(z.float(), approximate="tanh" if act_kind == 2 else "none").to(z.dtype)
+
+
+def moe_experts(h, idx, wts, w_gu, w_down, limit, alpha, shared, act_kind=0, weight_in=False, shared_scale=None):
     y = torch.zeros(h.shape, dtype=torch.float32)
     for e in idx.unique().tolist():
         tok, k = (idx == e).nonzero(as_tuple=True)
-        if act_kind == 0:
-            act = clamped_glu(F.linear(h[tok], w_gu[e]), limit, alpha)
-        elif act_kind == 3:
-            g, u = F.linear(h[tok], w_gu[e]).float().chunk(2, -1)
-            g, u = g.clamp(max=limit), u.clamp(-limit, limit)
-            act = (g * torch.sigmoid(alpha * g) * u).to(h.dtype)
-        else:
-            act = F.gelu(F.linear(h[tok], w_gu[e]).float(), approximate="tanh" if act_kind == 2 else "none").to(h.dtype)
-        y.index_add_(0, tok, wts[tok, k][:, None] * F.linear(act, w_down[e]).float())
+        w = wts[tok, k][:, None]
+        z = F.linear(h[tok], w_gu[e])
+        act = expert_act((z.float() * w).to(h.dtype) if weight_in else z, act_kind, limit, alpha)
+        out = F.linear(act, w_down[e]).float()
+        y.index_add_(0, tok, out if weight_in else w * out)
     if shared is not None:
-        y = y + shared.float()
+        y = y + shared.float() * (shared_scale[:, None] if shared_scale is not None else 1.0)
     return y.to(h.dtype)
 
 
@@ -437,8 +455,41 @@ def delta_gate_norm(o, g, norm_w, eps, dtype):
     return (_unit_rms(o, eps).reshape(T, H * D) * norm_w.float() * torch.sigmoid(g.float())).to(dtype)
 
 
-def relu_squared(z):
-    return torch.relu(z.float()).pow(2).to(z.dtype)
+def relu_squared(z, row_scale=None):
+    v = torch.relu(z.float()).pow(2)
+    return (v if row_scale is None else v * row_scale[:, None]).to(z.dtype)
+
+
+def layer_norm_residual(x, y, next_w, eps, dtype, ids, y2):
+    if ids is not None:
+        x = y[ids].float()
+    elif y is not None:
+        x += y.float()
+    if y2 is not None:
+        x += y2.float()
+    if next_w is None:
+        return x, None
+    d = x - x.mean(-1, keepdim=True)
+    return x, (d / torch.sqrt(d.pow(2).mean(-1, keepdim=True) + eps) * next_w.float()).to(dtype)
+
+
+def selective_scan(x, dt_pre, dt_bias, bc, b_off, c_off, A, D, z, state, ctx):
+    N = A.shape[1]
+    xf, zf, bcf = x.float(), z.float(), bc.float()
+    dt = F.softplus(dt_pre + dt_bias, threshold=50.0)
+    y = torch.empty(x.shape, dtype=torch.float32)
+    qs = ctx.qstart.tolist()
+    for b in range(ctx.num_seqs):
+        a, e = qs[b], qs[b + 1]
+        if e <= a:
+            continue
+        slot = int(ctx.seq_slot[b])
+        S = state[slot].clone() if int(ctx.seq_pos0[b]) > 0 else torch.zeros_like(state[slot])
+        for t in range(a, e):
+            S = torch.exp(dt[t][:, None] * A) * S + (dt[t] * xf[t])[:, None] * bcf[t, b_off:b_off + N][None, :]
+            y[t] = S @ bcf[t, c_off:c_off + N]
+        state[slot] = S
+    return ((y + D * xf) * F.silu(zf)).to(x.dtype)
 
 
 def group_norm_residual(x, y, post_w, groups, eps, dtype, next_w, ids, want_h):

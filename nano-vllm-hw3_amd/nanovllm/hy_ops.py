@@ -310,14 +310,79 @@ def delta_gate_norm(o, g, norm_w, eps, dtype):
     return out
 
 
-def relu_squared(z):
-    """max(z, 0)^2; z [T, F] may be a column slice of a wider product."""
-    if not z.is_cuda:
-        return cpu_ops.relu_squared(z)
-    _rows(z, "z")
+def relu_squared(z, row_scale=None, out=None):
+    """max(z, 0)^2, times row_scale[t] (f32 [T]) if given; z [T, F] and ``out`` may be column slices of wider matrices."""
     T, Fw = z.shape
-    out = torch.empty((T, Fw), dtype=z.dtype, device=z.device)
-    HM.check(HM.load().hm_relu_squared(HM.dtype_code(z.dtype), z.data_ptr(), z.stride(0), out.data_ptr(), T, Fw, _dev(z)))
+    if out is None:
+        out = torch.empty((T, Fw), dtype=z.dtype, device=z.device)
+    if not z.is_cuda:
+        out.copy_(cpu_ops.relu_squared(z, row_scale))
+        return out
+    _rows(z, "z")
+    _rows(out, "out")
+    assert out.shape == (T, Fw) and out.dtype == z.dtype and (row_scale is None or row_scale.dtype == torch.float32)
+    HM.check(HM.load().hm_relu_squared(HM.dtype_code(z.dtype), z.data_ptr(), z.stride(0), HM.ptr(row_scale), out.data_ptr(),
+                                       out.stride(0), T, Fw, _dev(z)))
+    return out
+
+
+def layer_norm_residual(x, y, next_w, eps, dtype, ids=None, y2=None, routed=None):
+    """The boundary between two blocks of a float32 residual x [T, W] whose blocks read a layer norm (weight, no bias) of it;
+    per token in one launch:
+      x <- x + y + y2     (ids given: x <- y[ids], y an embedding table; x may then be None and is made here)
+      routed = (prod, pair_row, weights or None), as moe_experts(combine=False) leaves it: the token's pairs are added too
+                          ((y, None, None): a sum that is already there)
+      next_w given:       h = (x - mean) / sqrt(mean((x - mean)^2) + eps) * next_w in ``dtype``.
+    Returns (x, h)."""
+    prod = pair_row = wts = None
+    if routed is not None:
+        if routed[1] is None:
+            assert y2 is None
+            y2 = routed[0]
+        else:
+            prod, pair_row, wts = routed
+    src = y if y is not None else x
+    if not src.is_cuda:
+        assert prod is None
+        return cpu_ops.layer_norm_residual(x, y, next_w, eps, dtype, ids, y2)
+    T = ids.numel() if ids is not None else src.shape[0]
+    W = src.shape[1]
+    if x is None:
+        x = torch.empty((T, W), dtype=torch.float32, device=src.device)
+    for a, name in ((y, "y"), (y2, "y2"), (prod, "prod")):
+        if a is not None:
+            HM.require_cuda(a, dtype, name)
+    h = torch.empty((T, W), dtype=dtype, device=x.device) if next_w is not None else None
+    HM.check(HM.load().hm_layer_norm_residual(HM.dtype_code(dtype), x.data_ptr(), HM.ptr(y), HM.ptr(ids), HM.ptr(y2), HM.ptr(prod),
+                                              HM.ptr(pair_row), HM.ptr(wts), pair_row.numel() // T if prod is not None else 0,
+                                              HM.ptr(next_w), float(eps), HM.ptr(h), T, W, _dev(x)))
+    return x, h
+
+
+def selective_scan(x, dt_pre, dt_bias, bc, b_off, c_off, A, D, z, state, ctx: StepContext, out=None):
+    """Selective scan over every sequence's portion, token after token, with a float32 state S [N] per channel:
+      dt = softplus(dt_pre + dt_bias);  S <- exp(dt A) S + dt x B;  out = (S . C + D x) silu(z)
+    x, z [T, channels] and bc (its columns b_off, c_off are B and C) may be column slices; dt_pre f32 [T, channels]; A f32
+    [channels, N], dt_bias and D f32 [channels].  state f32 [slots, channels, N] is read at a portion's start (zero at
+    position 0) and left at its end.  ``out`` [T, channels] (may be a column slice) takes the result."""
+    T, C = x.shape
+    N = A.shape[1]
+    if out is None:
+        out = torch.empty((T, C), dtype=x.dtype, device=x.device)
+    if not x.is_cuda:
+        out.copy_(cpu_ops.selective_scan(x, dt_pre, dt_bias, bc, b_off, c_off, A, D, z, state, ctx))
+        return out
+    for a, name in ((x, "x"), (dt_pre, "dt_pre"), (bc, "bc"), (z, "z"), (out, "out")):
+        _rows(a, name)
+    assert x.dtype == bc.dtype == z.dtype == out.dtype and dt_pre.dtype == A.dtype == D.dtype == dt_bias.dtype == torch.float32
+    assert dt_pre.shape == z.shape == out.shape == (T, C) and A.shape == (C, N) and A.is_contiguous()
+    assert dt_bias.numel() == D.numel() == C and bc.shape[0] == T and max(b_off, c_off) + N <= bc.shape[1]
+    assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (C, N)
+    HM.check(HM.load().hm_selective_scan(HM.dtype_code(x.dtype), x.data_ptr(), x.stride(0), dt_pre.data_ptr(), dt_pre.stride(0),
+                                         dt_bias.data_ptr(), bc.data_ptr(), bc.stride(0), b_off, c_off, A.data_ptr(), D.data_ptr(),
+                                         z.data_ptr(), z.stride(0), state.data_ptr(), ctx.qstart.data_ptr(), ctx.seq_pos0.data_ptr(),
+                                         ctx.seq_slot.data_ptr(), out.data_ptr(), out.stride(0), ctx.num_seqs, C, N,
+                                         max(int(ctx.max_q), 1), _dev(x)))
     return out
 
 

@@ -1,4 +1,5 @@
-"""Short causal convolution over time on every channel, added to its input ("canon" layer).  The last taps-1 inputs of
+"""Short causal convolution over time on every channel, added to its input ("canon" layer), or on its own with a bias and a
+SiLU behind it (``bias``, ``silu``, ``add_input`` = False: what a selective-scan mixer reads).  The last taps-1 inputs of
 every sequence are state: the engine gives each sequence a state slot, and one tensor holds the state of every
 (slot, layer run)."""
 import torch
@@ -8,11 +9,12 @@ from nanovllm import seq_ops
 
 
 class CausalTaps(nn.Module):
-    def __init__(self, width: int, taps: int):
+    def __init__(self, width: int, taps: int, bias: bool = False, silu: bool = False, add_input: bool = True):
         super().__init__()
-        self.taps = taps
+        self.taps, self.silu, self.add_input = taps, silu, add_input
+        self.bias = nn.Parameter(torch.zeros(width), requires_grad=False) if bias else None
         self.weight = nn.Parameter(torch.zeros(width, taps), requires_grad=False)     # [channel, tap]; tap taps-1 = now
         self.state = None          # [slots, runs, taps-1, width], shared by all layer runs (set by the cache allocation)
 
-    def forward(self, h, run: int):
-        return seq_ops.canon_conv(h, self.weight, self.state, run, seq_ops.get_step())
+    def forward(self, h, run: int = 0):
+        return seq_ops.short_conv(h, self.weight, self.state, run, seq_ops.get_step(), self.bias, self.silu, self.add_input)

@@ -135,7 +135,7 @@ class LilevikForCausalLM(nn.Module):
         elif isinstance(mx, LatentAttention) and rest == "mix.uk":
             mx.uk.data.copy_(tensor.view(mx.heads, mx.dim, mx.kv_rank))
         elif isinstance(mx, LatentAttention) and rest == "mix.uv":
-            mx.uv.data.copy_(tensor.view(mx.heads, mx.vdim, mx.kv_rank))
+            mx.uv.data.copy_(tensor.view(mx.heads, mx.vdim, mx.kv_rank).transpose(1, 2))
         else:
             e = re.fullmatch(r"mlp\.e(\d+)\.(gate|up|down)", rest)
             if not e or layer.mlp is None or int(e.group(1)) >= layer.mlp.experts:

@@ -128,7 +128,7 @@ class PasizenForCausalLM(nn.Module):
         elif rest == "mix.uk":
             mx.uk.data.copy_(tensor.view(mx.heads, mx.dim, mx.kv_rank))
         elif rest == "mix.uv":
-            mx.uv.data.copy_(tensor.view(mx.heads, mx.vdim, mx.kv_rank))
+            mx.uv.data.copy_(tensor.view(mx.heads, mx.vdim, mx.kv_rank).transpose(1, 2))
         elif rest in ("mlp.shared.gate", "mlp.shared.up"):
             sh = layer.mlp.shared
             sh.gate_up.data[(sh.ff if rest.endswith("up") else 0):][:sh.ff].copy_(tensor)

@@ -71,21 +71,21 @@ def stream_step(X, y, mix, out, w_in, norm_w, eps, dtype):
     return h
 
 
-def canon_conv(h, w, state, run, ctx: StepContext):
-    """h + causal_conv(h) per channel with the sequence's carried inputs; then the state takes this step's last inputs.
-    h [T, W], w [W, taps], state [slots, runs, taps-1, W]."""
-    T, W = h.shape
+def short_conv(x, w, state, run, ctx: StepContext, bias=None, silu=False, add_input=False):
+    """Causal convolution per channel over the sequence's carried inputs and this step's, + bias, then SiLU if asked for;
+    ``add_input``: the input is added to the result.  The state takes the step's last inputs (same launch).
+    x [T, W] (rows may be a column slice), w [W, taps], bias [W], state [slots, runs, taps-1, W] -> dense [T, W]."""
+    T, W = x.shape
     taps = w.shape[1]
-    if not h.is_cuda:
-        return cpu_ops.canon_conv(h, w, state, run, ctx)
-    SM.require_cuda(h, w.dtype, "h")
-    out = torch.empty_like(h)
-    lib, code, runs = SM.load(), SM.dtype_code(h.dtype), state.shape[1]
-    SM.check(lib.sm_canon_conv(code, h.data_ptr(), w.data_ptr(), state.data_ptr(), run, runs, ctx.tok_seq.data_ptr(),
-                               ctx.tok_pos.data_ptr(), ctx.qstart.data_ptr(), ctx.seq_slot.data_ptr(), out.data_ptr(), T, W,
-                               taps, _dev(h)))
-    SM.check(lib.sm_canon_update(code, h.data_ptr(), state.data_ptr(), run, runs, ctx.qstart.data_ptr(),
-                                 ctx.seq_slot.data_ptr(), ctx.num_seqs, W, taps, _dev(h)))
+    if not x.is_cuda:
+        return cpu_ops.short_conv(x, w, state, run, ctx, bias, silu, add_input)
+    assert x.stride(1) == 1 and x.dtype == w.dtype and w.is_contiguous() and (bias is None or bias.dtype == w.dtype)
+    assert taps == 1 or (state.is_contiguous() and state.dtype == x.dtype and state.shape[2:] == (taps - 1, W))
+    out = torch.empty((T, W), dtype=x.dtype, device=x.device)
+    SM.check(SM.load().sm_short_conv(SM.dtype_code(x.dtype), x.data_ptr(), x.stride(0), w.data_ptr(), SM.ptr(bias), int(bool(silu)),
+                                     int(bool(add_input)), SM.ptr(state), run, state.shape[1] if state is not None else run + 1,
+                                     ctx.qstart.data_ptr(), ctx.seq_pos0.data_ptr(), ctx.seq_slot.data_ptr(), out.data_ptr(),
+                                     ctx.num_seqs, int(ctx.max_q), W, taps, _dev(x)))
     return out
 
 
@@ -112,32 +112,39 @@ def rms_norm_rows(x, w, eps):
     return out
 
 
-def latent_rope_store(x, w, eps, q, qa, inv_freq, rot_dims, H, D, R, Rd, cache, ctx: StepContext):
+def latent_rope_store(x, w, eps, q, qa, inv_freq, rot_dims, H, D, R, Rd, cache, ctx: StepContext, rot_mag=1.0):
     """A latent with a rotated key part.  x [T, R + Rd] (rows may be a column slice): rms_norm(x[:, :R]) * w and x[:, R:]
     with its first rot_dims channels turned by position * inv_freq (channel 2i pairs with 2i + 1) are stored as the
     tokens' rows of ``cache`` [blocks, block_size, R + Rd].  q [T, H * (D + Rd)] (rows may be a slice): every head's last
-    Rd channels, turned the same way, go to qa[:, :, R:] (qa [T, H, R + Rd]; its first R columns are the caller's)."""
-    if not x.is_cuda:
-        return cpu_ops.latent_rope_store(x, w, eps, q, qa, inv_freq, rot_dims, H, D, R, Rd, cache, ctx)
-    T = x.shape[0]
-    assert x.stride(1) == 1 and q.stride(1) == 1 and qa.is_contiguous() and x.dtype == cache.dtype == w.dtype == q.dtype == qa.dtype
-    assert x.shape[1] == R + Rd and q.shape[1] == H * (D + Rd) and qa.shape == (T, H, R + Rd) and cache.shape[2] == R + Rd
-    SM.check(SM.load().sm_latent_rope_store(SM.dtype_code(x.dtype), x.data_ptr(), x.stride(0), w.data_ptr(), eps, q.data_ptr(),
-                                            q.stride(0), qa.data_ptr(), SM.ptr(inv_freq), rot_dims, ctx.tok_pos.data_ptr(),
-                                            cache.data_ptr(), ctx.slot_mapping.data_ptr(), T, H, D, R, Rd, _dev(x)))
+    Rd channels, turned the same way, go to qa[:, :, R:] (qa [T, H, R + Rd]; its first R columns are the caller's).
+    ``rot_mag`` multiplies every cosine and sine.  x None: only the queries are turned (another layer stores the rows)."""
+    if not q.is_cuda:
+        return cpu_ops.latent_rope_store(x, w, eps, q, qa, inv_freq, rot_dims, H, D, R, Rd, cache, ctx, rot_mag)
+    T = q.shape[0]
+    assert q.stride(1) == 1 and qa.is_contiguous() and q.dtype == qa.dtype
+    assert q.shape[1] == H * (D + Rd) and qa.shape == (T, H, R + Rd)
+    if x is not None:
+        assert x.stride(1) == 1 and x.dtype == cache.dtype == w.dtype == q.dtype
+        assert x.shape == (T, R + Rd) and cache.shape[2] == R + Rd
+    SM.check(SM.load().sm_latent_rope_store(SM.dtype_code(q.dtype), SM.ptr(x), x.stride(0) if x is not None else 0, SM.ptr(w), eps,
+                                            q.data_ptr(), q.stride(0), qa.data_ptr(), SM.ptr(inv_freq), rot_dims,
+                                            ctx.tok_pos.data_ptr(), SM.ptr(cache) if x is not None else None,
+                                            ctx.slot_mapping.data_ptr(), T, H, D, R, Rd, float(rot_mag), _dev(q)))
 
 
 USE_TILES = True       # bf16 latent attention on the matrix cores where the shape allows (tests compare both forms)
 
 
-def latent_attention(q, cache, ctx: StepContext, scale, force_rows=False, value_cols=0, window=0):
+def latent_attention(q, cache, ctx: StepContext, scale, force_rows=False, value_cols=0, window=0, sink=None):
     """Absorbed queries q [T, H, R] over the paged latent cache [blocks, block_size, R], causal inside each sequence.
     A cache row is the key; its first ``value_cols`` columns are the value (0 = all of it) -> [T, H, value_cols or R].
-    ``window`` > 0: the token at position i sees only the keys j with i - j < window."""
+    ``window`` > 0: the token at position i sees only the keys j with i - j < window.  ``sink`` f32 [H]: one more term
+    exp(sink[h]) in the softmax denominator, without a key and a value, not scaled."""
+    assert sink is None or (sink.dtype == torch.float32 and sink.numel() == q.shape[1])
     T, H, R = q.shape
     RV = value_cols or R
     if not q.is_cuda:
-        return cpu_ops.latent_attention(q, cache, ctx, scale, RV, window)
+        return cpu_ops.latent_attention(q, cache, ctx, scale, RV, window, sink)
     SM.require_cuda(q, cache.dtype, "q")
     o = torch.empty((T, H, RV), dtype=q.dtype, device=q.device)
     lib = SM.load()
@@ -148,15 +155,15 @@ def latent_attention(q, cache, ctx: StepContext, scale, force_rows=False, value_
         splits = decode_splits(ctx.num_seqs, min(mb * bs, window + 64) if window > 0 else mb * bs)
         ws, n = SM.decode_workspace.get(q.device, lib.sm_latent_decode_workspace_bytes(T, H, R, splits))
         SM.check(lib.sm_latent_attn_decode(q.data_ptr(), cache.data_ptr(), ctx.block_tables.data_ptr(), ctx.ctx_lens.data_ptr(),
-                                           o.data_ptr(), scale, T, H, R, bs, mb, splits, ws, n, RV, int(window), _dev(q)))
+                                           o.data_ptr(), scale, T, H, R, bs, mb, splits, ws, n, RV, int(window), SM.ptr(sink), _dev(q)))
     elif tiles_ok:
         SM.check(lib.sm_latent_attn_tiles(q.data_ptr(), cache.data_ptr(), ctx.block_tables.data_ptr(), ctx.qstart.data_ptr(),
                                           ctx.seq_pos0.data_ptr(), o.data_ptr(), scale, ctx.num_seqs, ctx.max_q, H, R, bs, mb,
-                                          RV, int(window), _dev(q)))
+                                          RV, int(window), SM.ptr(sink), _dev(q)))
     else:
         SM.check(lib.sm_latent_attn_rows(SM.dtype_code(q.dtype), q.data_ptr(), cache.data_ptr(), ctx.block_tables.data_ptr(),
                                          ctx.tok_seq.data_ptr(), ctx.tok_pos.data_ptr(), o.data_ptr(), scale, T, H, R, bs, mb,
-                                         RV, int(window), _dev(q)))
+                                         RV, int(window), SM.ptr(sink), _dev(q)))
     return o
 
 
@@ -178,6 +185,21 @@ def poly_norm(z, coef, eps):
     return out
 
 
+def gated_act(gu, act_kind, limit=float("inf"), alpha=1.0, out=None):
+    """gu [T, 2F] = gate | up (rows may be a column slice) -> the gated activation ``act_kind`` (one of GATED_ACTS), e.g.
+    ACT_GELU_TANH_GLU: gelu_tanh(gate) * up.  ``out`` [T, F] (rows may be a column slice) takes the result."""
+    T, F2 = gu.shape
+    if out is None:
+        out = torch.empty((T, F2 // 2), dtype=gu.dtype, device=gu.device)
+    if not gu.is_cuda:
+        out.copy_(cpu_ops.expert_act(gu, act_kind, limit, alpha))
+        return out
+    assert gu.stride(1) == 1 and out.stride(1) == 1 and out.dtype == gu.dtype and out.shape == (T, F2 // 2)
+    SM.check(SM.load().sm_gated_act(SM.dtype_code(gu.dtype), gu.data_ptr(), gu.stride(0), int(act_kind), limit, alpha, out.data_ptr(),
+                                    out.stride(0), T, F2 // 2, _dev(gu)))
+    return out
+
+
 def clamped_glu(gu, limit, alpha=1.702):
     """gu [T, 2F] = gate | up -> min(g, limit) * sigmoid(alpha * min(g, limit)) * (clamp(u, +-limit) + 1)."""
     if not gu.is_cuda:
@@ -190,18 +212,21 @@ def clamped_glu(gu, limit, alpha=1.702):
 
 
 ROUTE_SOFTMAX, ROUTE_SIGMOID = 0, 1
-ACT_CLAMPED_GLU, ACT_GELU, ACT_GELU_TANH, ACT_SILU_GLU = 0, 1, 2, 3
-GATED_ACTS = (ACT_CLAMPED_GLU, ACT_SILU_GLU)      # experts with gate and up rows
+ACT_CLAMPED_GLU, ACT_GELU, ACT_GELU_TANH, ACT_SILU_GLU, ACT_RELU_SQ, ACT_GELU_TANH_GLU = 0, 1, 2, 3, 4, 5
+GATED_ACTS = (ACT_CLAMPED_GLU, ACT_SILU_GLU, ACT_GELU_TANH_GLU)      # those of a gate and an up product
 
 
-def moe_route(h, router_w, top, groups=1, keep=1, score=ROUTE_SOFTMAX, correction=None, group_top=1, renorm=True, bias=None):
+def moe_route(h, router_w, top, groups=1, keep=1, score=ROUTE_SOFTMAX, correction=None, group_top=1, renorm=True, bias=None,
+              gate_w=None):
     """Router with group-limited top-k: (idx int32 [T, top], weights f32 [T, top]); router_w f32 [E, W].  Scores are the
     softmax or the sigmoid of the float32 logits; ``correction`` f32 [E] is added for the CHOICE only (groups and
     experts), the weights stay the scores; a group scores the sum of its ``group_top`` largest choice scores (1 = its
     maximum); ``renorm``: the chosen weights are divided by their sum.  ``bias`` f32 [E] is added to the logits (softmax
-    scores with ``renorm`` are then the softmax over the chosen experts' logits)."""
+    scores with ``renorm`` are then the softmax over the chosen experts' logits).  ``gate_w`` f32 [W]: a third result
+    sigmoid(gate_w . h) f32 [T] from the same pass over h."""
     if not h.is_cuda:
-        return cpu_ops.moe_route(h, router_w, top, groups, keep, score, correction, group_top, renorm, bias)
+        res = cpu_ops.moe_route(h, router_w, top, groups, keep, score, correction, group_top, renorm, bias)
+        return res if gate_w is None else (*res, torch.sigmoid(h.float() @ gate_w.float()))
     if bias is not None:
         SM.require_cuda(bias, torch.float32, "bias")
     if correction is not None:
@@ -212,10 +237,15 @@ def moe_route(h, router_w, top, groups=1, keep=1, score=ROUTE_SOFTMAX, correctio
     E = router_w.shape[0]
     idx = torch.empty((T, top), dtype=torch.int32, device=h.device)
     wts = torch.empty((T, top), dtype=torch.float32, device=h.device)
+    gate = None
+    if gate_w is not None:
+        SM.require_cuda(gate_w, torch.float32, "gate_w")
+        assert gate_w.numel() == W
+        gate = torch.empty((T,), dtype=torch.float32, device=h.device)
     SM.check(SM.load().sm_moe_route(SM.dtype_code(h.dtype), h.data_ptr(), router_w.data_ptr(), idx.data_ptr(), wts.data_ptr(),
                                     T, W, E, top, groups, keep, int(score), SM.ptr(correction), int(group_top), int(bool(renorm)),
-                                    SM.ptr(bias), _dev(h)))
-    return idx, wts
+                                    SM.ptr(bias), SM.ptr(gate_w), SM.ptr(gate), _dev(h)))
+    return (idx, wts) if gate is None else (idx, wts, gate)
 
 
 TILES128_MIN_ROWS_PER_EXPERT = 64
@@ -234,16 +264,24 @@ def tile_expert_weights(w, parts=1):
     return x.contiguous()
 
 
-def moe_experts(h, idx, wts, w_gu, w_down, limit, alpha=1.702, shared=None, form=None, tiled=None, act_kind=ACT_CLAMPED_GLU):
+def moe_experts(h, idx, wts, w_gu, w_down, limit, alpha=1.702, shared=None, form=None, tiled=None, act_kind=ACT_CLAMPED_GLU,
+                weight_in=False, shared_scale=None, combine=True):
     """y[t] = sum_k wts[t, k] * expert_{idx[t, k]}(h[t]) (+ shared[t]); w_gu [E, 2F, W] (gate rows then up rows),
     w_down [E, W, F]; an expert is a clamped GLU between its two products.  ``form``: "pairs" | "grouped" | "tiles128"
     forces one; by default float32 runs pair by pair and bf16 grouped by expert on the matrix cores, in tiles of 32 rows
     for small groups (decode) and of 128 rows for large ones (prefill).  ``tiled`` = (tile_expert_weights(w_gu, 2),
     tile_expert_weights(w_down)), what the grouped forms read (made here when the caller does not keep them).
     ``act_kind`` = ACT_GELU / ACT_GELU_TANH: an expert is down(gelu(up h)) instead, w_gu is [E, F, W] (tiled in one part);
-    ACT_SILU_GLU: the gated form g sigmoid(alpha g) u without the one and, with limit = inf and alpha = 1, silu(gate) * up."""
+    ACT_SILU_GLU: the gated form g sigmoid(alpha g) u without the one and, with limit = inf and alpha = 1, silu(gate) * up;
+    ACT_GELU_TANH_GLU: gelu_tanh(gate) * up; ACT_RELU_SQ: down(max(up h, 0)^2).
+    ``weight_in``: the weight multiplies what an expert reads, y[t] = sum_k expert(wts[t, k] h[t]).  ``shared_scale`` f32 [T]:
+    a factor on shared[t].  ``combine`` False (without ``shared``): the sum may be left to the caller: returns
+    (prod, pair_row, weights or None) with y[t] = sum_k weights[t, k] prod[pair_row[t, k]], or (y, None, None) where the form
+    has summed already."""
+    assert combine or shared is None
     if not h.is_cuda:
-        return cpu_ops.moe_experts(h, idx, wts, w_gu, w_down, limit, alpha, shared, act_kind)
+        y = cpu_ops.moe_experts(h, idx, wts, w_gu, w_down, limit, alpha, shared, act_kind, weight_in, shared_scale)
+        return y if combine else (y, None, None)
     parts = 2 if act_kind in GATED_ACTS else 1
     assert w_gu.shape[1] == parts * w_down.shape[2]
     SM.require_cuda(h, w_gu.dtype, "h")
@@ -261,20 +299,20 @@ def moe_experts(h, idx, wts, w_gu, w_down, limit, alpha=1.702, shared=None, form
         n = lib.sm_moe_grouped_tiles(T, top, E) if form == "grouped" else lib.sm_moe_tiles128_count(T, top, E)
         ints = torch.empty(rows * n + n + T * top, dtype=torch.int32, device=h.device)
         row_pair, tile_expert, pair_row = ints[:rows * n], ints[rows * n:rows * n + n], ints[rows * n + n:]
-        y = torch.empty_like(h)
+        y = torch.empty_like(h) if combine else None
         prod = torch.empty((rows * n, W), dtype=h.dtype, device=h.device)
         act = torch.empty((rows * n, F), dtype=h.dtype, device=h.device)
         fn = lib.sm_moe_grouped if form == "grouped" else lib.sm_moe_tiles128
         t_gu, t_down = tiled if tiled is not None else (tile_expert_weights(w_gu, parts), tile_expert_weights(w_down))
-        SM.check(fn(h.data_ptr(), idx.data_ptr(), wts.data_ptr(), t_gu.data_ptr(), t_down.data_ptr(), SM.ptr(shared), limit, alpha,
-                    int(act_kind), y.data_ptr(), T, top, E, W, F, row_pair.data_ptr(), tile_expert.data_ptr(), pair_row.data_ptr(),
+        SM.check(fn(h.data_ptr(), idx.data_ptr(), wts.data_ptr(), t_gu.data_ptr(), t_down.data_ptr(), SM.ptr(shared),
+                    SM.ptr(shared_scale), int(bool(weight_in)), limit, alpha, int(act_kind), SM.ptr(y), T, top, E, W, F, row_pair.data_ptr(), tile_expert.data_ptr(), pair_row.data_ptr(),
                     act.data_ptr(), prod.data_ptr(), _dev(h)))
-        return y
+        return y if combine else (prod, pair_row, None if weight_in else wts)
     assert form == "pairs", form
     act = torch.empty((T * top, F), dtype=h.dtype, device=h.device)
     y = torch.empty_like(h)
     SM.check(lib.sm_moe_pairs_gate_up(code, h.data_ptr(), idx.data_ptr(), w_gu.data_ptr(), limit, alpha, int(act_kind),
-                                      act.data_ptr(), T, top, W, F, _dev(h)))
-    SM.check(lib.sm_moe_pairs_down(code, act.data_ptr(), idx.data_ptr(), wts.data_ptr(), w_down.data_ptr(), SM.ptr(shared),
-                                   y.data_ptr(), T, top, W, F, _dev(h)))
-    return y
+                                      wts.data_ptr() if weight_in else None, act.data_ptr(), T, top, W, F, _dev(h)))
+    SM.check(lib.sm_moe_pairs_down(code, act.data_ptr(), idx.data_ptr(), None if weight_in else wts.data_ptr(), w_down.data_ptr(),
+                                   SM.ptr(shared), SM.ptr(shared_scale), y.data_ptr(), T, top, W, F, _dev(h)))
+    return y if combine else (y, None, None)

@@ -234,7 +234,7 @@ def kernel_table(width=2048, heads=16, rank=256, ff=6144, T=8192, seq=1024, B=64
     # ---- short convolution | Qwen3 has none: its elementwise launch (SiLU * mul) is the like kernel
     h, cw = r(T, width), r(width, taps)
     state = torch.zeros(nseq, 1, taps - 1, width, device=dev, dtype=bf)
-    add("sm_canon_conv+update (T=%d)" % T, "ql_silu_mul", _event_time(lambda: seq_ops.canon_conv(h, cw, state, 0, pre)), bytes_=T * width * 4)
+    add("sm_short_conv, input added (T=%d)" % T, "ql_silu_mul", _event_time(lambda: seq_ops.short_conv(h, cw, state, 0, pre, add_input=True)), bytes_=T * width * 4)
     gu = r(T, 2 * ff)
     add("ql_silu_mul (T=%d)" % T, "-", _event_time(lambda: ops.silu_mul(gu)), bytes_=T * ff * 6)
     # ---- activations

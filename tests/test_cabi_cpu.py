@@ -125,16 +125,18 @@ def test_seqmix_argument_validation_needs_no_gpu():
     assert lib.sm_stream_step(7, one, one, one, one, one, one, 1e-5, one, 4, 2, 64, None) == -1          # unknown dtype
     assert lib.sm_stream_step(1, one, one, one, one, one, one, 1e-5, one, 4, 9, 64, None) == -2          # too many streams
     assert b"streams" in lib.sm_last_error()
-    assert lib.sm_canon_conv(1, one, one, one, 3, 3, one, one, one, one, one, 4, 64, 4, None) == -1      # run >= runs
-    assert lib.sm_latent_attn_tiles(one, one, one, one, one, one, 0.1, 2, 8, 4, 36, 64, 4, 0, 0, None) == -2   # R % 8
-    assert lib.sm_latent_attn_tiles(one, one, one, one, one, one, 0.1, 2, 8, 4, 64, 48, 4, 0, 0, None) == -2   # block % 64
-    assert lib.sm_latent_attn_tiles(one, one, one, one, one, one, 0.1, 2, 8, 4, 64, 64, 4, 72, 0, None) == -1   # values wider than the row
-    assert lib.sm_latent_rope_store(1, one, 40, one, 1e-5, one, 96, one, one, 12, one, one, one, 4, 2, 16, 32, 8, None) == -1   # rotation wider than the part
-    assert lib.sm_latent_attn_decode(one, one, one, one, one, 0.1, 2, 4, 64, 64, 4, 2, one, 16, 0, 0, None) == -3   # workspace
-    assert lib.sm_moe_route(1, one, one, one, one, 4, 64, 8, 3, 4, 1, 0, None, 1, 1, None, None) == -2    # top > keep * E/groups
-    assert lib.sm_moe_route(1, one, one, one, one, 4, 64, 8, 2, 4, 2, 5, None, 1, 1, None, None) == -1    # unknown score function
-    assert lib.sm_moe_grouped(one, one, one, one, one, None, 1.0, 1.7, 0, one, 4, 2, 8, 60, 64, one, one, one, one, one, None) == -2
-    assert lib.sm_moe_grouped(one, one, one, one, one, None, 1.0, 1.7, 9, one, 4, 2, 8, 64, 64, one, one, one, one, one, None) == -1   # unknown activation
+    assert lib.sm_short_conv(1, one, 64, one, None, 0, 1, one, 3, 3, one, one, one, one, 2, 4, 64, 4, None) == -1      # run >= runs
+    assert lib.sm_latent_attn_tiles(one, one, one, one, one, one, 0.1, 2, 8, 4, 36, 64, 4, 0, 0, None, None) == -2   # R % 8
+    assert lib.sm_latent_attn_tiles(one, one, one, one, one, one, 0.1, 2, 8, 4, 64, 48, 4, 0, 0, None, None) == -2   # block % 64
+    assert lib.sm_latent_attn_tiles(one, one, one, one, one, one, 0.1, 2, 8, 4, 64, 64, 4, 72, 0, None, None) == -1   # values wider than the row
+    assert lib.sm_latent_rope_store(1, one, 40, one, 1e-5, one, 96, one, one, 12, one, one, one, 4, 2, 16, 32, 8, 1.0, None) == -1   # rotation wider than the part
+    assert lib.sm_latent_attn_decode(one, one, one, one, one, 0.1, 2, 4, 64, 64, 4, 2, one, 16, 0, 0, None, None) == -3   # workspace
+    assert lib.sm_moe_route(1, one, one, one, one, 4, 64, 8, 3, 4, 1, 0, None, 1, 1, None, None, None, None) == -2    # top > keep * E/groups
+    assert lib.sm_moe_route(1, one, one, one, one, 4, 64, 8, 2, 4, 2, 5, None, 1, 1, None, None, None, None) == -1    # unknown score function
+    assert lib.sm_moe_route(1, one, one, one, one, 4, 64, 8, 2, 1, 1, 1, None, 1, 0, None, one, None, None) == -1    # a gate without its result
+    assert lib.sm_gated_act(1, one, 64, 1, 1.0, 1.0, one, 32, 4, 32, None) == -1     # not a gated activation
+    assert lib.sm_moe_grouped(one, one, one, one, one, None, None, 0, 1.0, 1.7, 0, one, 4, 2, 8, 60, 64, one, one, one, one, one, None) == -2
+    assert lib.sm_moe_grouped(one, one, one, one, one, None, None, 0, 1.0, 1.7, 9, one, 4, 2, 8, 64, 64, one, one, one, one, one, None) == -1   # unknown activation
 
 
 # ---- libhymix (include/hymix.h) ----------------------------------------------------------------------------------------

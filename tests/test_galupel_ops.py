@@ -191,7 +191,7 @@ def run_latent(device, dtype, H, D, Rd, V, R, window, dims, lengths, cuts, seed=
     mod.qc_proj.data.copy_(torch.cat([p["mix.q"], p["mix.dkv"]]))
     mod.latent_norm.data.copy_(p["mix.dkv.norm"])
     mod.uk.data.copy_(p["mix.uk"].view(H, D, R))
-    mod.uv.data.copy_(p["mix.uv"].view(H, V, R))
+    mod.uv.data.copy_(p["mix.uv"].view(H, V, R).transpose(1, 2))
     mod.o_proj.data.copy_(p["mix.o"])
     mod.to(device)
     m = dict(heads=H, dim=D, rot_dim=Rd, vdim=V, kv_rank=R, scale=scale, rot=dict(dims=dims, base=base), mask=dict(size=window))

@@ -228,7 +228,7 @@ def test_latent_attention_with_query_latent(device, dtype, H, D, Rd, V, R, Q):
     mod.uq.data.copy_(p["mix.uq"])
     mod.latent_norm.data.copy_(p["mix.dkv.norm"])
     mod.uk.data.copy_(p["mix.uk"].view(H, D, R))
-    mod.uv.data.copy_(p["mix.uv"].view(H, V, R))
+    mod.uv.data.copy_(p["mix.uv"].view(H, V, R).transpose(1, 2))
     mod.o_proj.data.copy_(p["mix.o"])
     mod.to(device)
     m = dict(heads=H, dim=D, rot_dim=Rd, vdim=V, kv_rank=R, q_rank=Q, scale=scale, rot=dict(dims=Rd, base=50.0))

@@ -110,7 +110,7 @@ def test_canon_conv_portions_and_state(device, dtype, taps):
         portions = [(cuts[b][step][0], cuts[b][step][1] - cuts[b][step][0]) for b in act]
         ctx = step_context(portions, 64, [[0]] * len(act), [[2, 0][b] for b in act], device)
         h = torch.cat([hs[b][cuts[b][step][0]:cuts[b][step][1]] for b in act]).to(device, dtype)
-        out = seq_ops.canon_conv(h, w.to(device, dtype), state, 1, ctx)
+        out = seq_ops.short_conv(h, w.to(device, dtype), state, 1, ctx, add_input=True)
         want = torch.cat([ref[b][cuts[b][step][0]:cuts[b][step][1]] for b in act])
         assert torch.allclose(out.float().cpu(), want, **tol(dtype, 4)), (taps, step)
         step += 1
