@@ -2,7 +2,8 @@
 GPU), and the time of every libseqmix / libhymix kernel beside the like kernel of the Qwen3 path with both against their
 rooflines; for the Galupel family the comparison is with Pasizen, the closest of the three (latent attention and routed
 experts), and its kernels stand beside the forms of the same kernels that Pasizen and Lipelix run; for the Lilevik
-family with Galupel (latent attention, masked attention, routed experts) and Lipelix (a recurrent mixer).  Used by
+family with Galupel (latent attention, masked attention, routed experts) and Lipelix (a recurrent mixer); for the Tafopel
+family with Lilevik (latent attention behind a query latent, a recurrent mixer, routed experts).  Used by
 ``bench.py --families [--family NAME]``; prints one JSON object."""
 import json
 import os
@@ -90,6 +91,22 @@ def lilevik_config(width, heads, ff, layers, rank):
                 layers=[dict(type=kinds[i % 4][0], mixer=kinds[i % 4][1], mlp=moe) for i in range(layers)])
 
 
+def tafopel_config(width, heads, ff, layers, rank):
+    """Selective scan (2 x width channels of 16 states, 4 taps, step sizes of rank width / 16), latent attention as wide as
+    Lilevik's at the size (query latent of 3 x rank, cache row rank - 64 + 64, a table stretched 4x, sinks), a second scan
+    layer, and a latent layer that reads the first one's rows.  The first layer's feed-forward is dense (tanh-GELU gate, ff);
+    the others have 16 squared-ReLU experts of ff/4 with 4 chosen and a shared one of ff/4."""
+    scan = dict(inner=2 * width, state=16, conv=4, dt_rank=width // 16)
+    lat = dict(heads=heads, dim=128, rot_dim=64, vdim=128, kv_rank=rank - 64, q_rank=3 * rank, scale=192 ** -0.5,
+               rot=dict(dims=64, base=10000.0, scaling=dict(factor=4.0, original=2048, fast=32.0, slow=1.0)))
+    moe = dict(kind="moe", expert=dict(ff=ff // 4), router=dict(experts=16, top=4), shared=dict(ff=ff // 4))
+    specs = []
+    for i in range(layers):
+        kind, m = ("mamba1", scan) if i % 2 == 0 else ("latent_attention", dict(lat, kv_from=i - 2) if i % 4 == 3 else lat)
+        specs.append(dict(type=kind, mixer=m, mlp=moe if i else dict(kind="dense", ff=ff)))
+    return dict(architecture="Tafopel", vocab=VOCAB, width=width, norm=dict(eps=1e-5), max_positions=8192, layers=specs)
+
+
 def _model_dir(cfg):
     d = tempfile.mkdtemp(prefix="family_bench_")
     with open(os.path.join(d, "config.json"), "w") as f:
@@ -116,7 +133,8 @@ def engine_throughput(family, size, prefill_seqs=8, prefill_len=1024, decode_seq
     cfg = (pasizen_config(width, heads, ff, layers, rank) if family == "pasizen" else
            lipelix_config(width, heads, ff, layers) if family == "lipelix" else
            galupel_config(width, heads, ff, layers, rank) if family == "galupel" else
-           lilevik_config(width, heads, ff, layers, rank) if family == "lilevik" else qwen3_config(width, heads, ff, layers))
+           lilevik_config(width, heads, ff, layers, rank) if family == "lilevik" else
+           tafopel_config(width, heads, ff, layers, rank) if family == "tafopel" else qwen3_config(width, heads, ff, layers))
     llm = LLM(_model_dir(cfg), load_format="dummy", enforce_eager=False, max_model_len=2048,
               max_num_seqs=decode_seqs, max_num_batched_tokens=prefill_seqs * prefill_len, gpu_memory_utilization=0.5)
     g = torch.Generator().manual_seed(0)
@@ -713,13 +731,167 @@ def lilevik_kernel_table(width=2048, heads=16, rank=256, ff=6144, T=8192, seq=10
     return rows
 
 
+def tafopel_kernel_table(width=2048, heads=16, rank=256, ff=6144, T=8192, seq=1024, B=64, ctx=1024):
+    """Seconds per launch of every kernel form the Tafopel family runs at a layer's size, its bound and the fraction of it
+    reached; beside each the form of the like kernel that Lilevik runs (`like`)."""
+    from nanovllm import hy_ops, seq_ops
+    from nanovllm.layers.f32_product import F32Product
+    dev, bf = "cuda", torch.bfloat16
+    rows = []
+
+    def add(name, like, sec, bytes_=0, flops=0, peak=MFMA_TFLOPS):
+        bound = max(bytes_ / (HBM_GBPS * 1e9), flops / (peak * 1e12))
+        rows.append(dict(kernel=name, like=like, us=round(sec * 1e6, 1), bound_us=round(bound * 1e6, 1),
+                         of_roofline=round(bound / sec, 3), bound="flops" if flops / (peak * 1e12) > bytes_ / (HBM_GBPS * 1e9) else "bytes"))
+    r = lambda *s: torch.randn(*s, device=dev).to(bf)  # noqa: E731
+    nseq, bs, D, Rd = T // seq, 64, 128, 64
+    R = rank - Rd
+    import numpy as np
+
+    def context(portions):
+        tables, nxt = [], 0
+        for p0, n in portions:
+            nb = (p0 + n + bs - 1) // bs
+            tables.append(list(range(nxt, nxt + nb)))
+            nxt += nb
+        tok_seq = np.concatenate([np.full(n, b) for b, (_, n) in enumerate(portions)])
+        tok_pos = np.concatenate([np.arange(p0, p0 + n) for p0, n in portions])
+        slot = np.concatenate([np.asarray(tables[b])[np.arange(p0, p0 + n) // bs] * bs + np.arange(p0, p0 + n) % bs
+                               for b, (p0, n) in enumerate(portions)])
+        mb = max(len(t) for t in tables)
+        bt = np.zeros((len(portions), mb), dtype=np.int32)
+        for b, t in enumerate(tables):
+            bt[b, :len(t)] = t
+        qs = np.concatenate([[0], np.cumsum([n for _, n in portions])])
+        i32 = lambda v: torch.tensor(np.asarray(v), dtype=torch.int32, device=dev)  # noqa: E731
+        return seq_ops.StepContext(tok_seq=i32(tok_seq), tok_pos=i32(tok_pos), qstart=i32(qs), seq_pos0=i32([p for p, _ in portions]),
+                                   ctx_lens=i32([p + n for p, n in portions]), seq_slot=i32(list(range(len(portions)))),
+                                   slot_mapping=i32(slot), block_tables=i32(bt), num_seqs=len(portions), num_tokens=int(qs[-1]),
+                                   max_q=max(n for _, n in portions), block_size=bs, qstart_host=qs.tolist()), nxt
+    pre, nblk_p = context([(0, seq)] * nseq)
+    dec, nblk_d = context([(ctx - 1, 1)] * B)
+    nblk = max(nblk_p, nblk_d)
+    # ---- residual boundary: add + layer norm, with and without the experts' rows | Lilevik: tanh norms
+    x, y, nw = torch.randn(T, width, device=dev), r(T, width), r(width)
+    add("hm_layer_norm_residual (T=%d)" % T, "hm_dyt_residual", _event_time(lambda: hy_ops.layer_norm_residual(x, y, nw, 1e-5, bf)),
+        bytes_=T * width * (8 + 2 + 2))
+    top, E, F = 4, 16, ff // 4
+    prod = r(T * top + 128 * E, width)
+    pair_row = torch.randperm(T * top, device=dev).int()
+    add("hm_layer_norm_residual + expert rows, top %d (T=%d)" % (top, T), "sm_moe_combine + hm_dyt_residual",
+        _event_time(lambda: hy_ops.layer_norm_residual(x, y, nw, 1e-5, bf, routed=(prod, pair_row, None))), bytes_=T * width * (8 + 2 + 2 + 2 * top))
+    n1, n2 = (r(width), r(width), torch.rand(1, device=dev)), (r(width), r(width), torch.rand(1, device=dev))
+    add("hm_dyt_residual (T=%d)" % T, "-", _event_time(lambda: hy_ops.dyt_residual(x, y, n1, n2, bf)), bytes_=T * width * (8 + 2 + 2))
+    # ---- selective scan: 2 x width channels of 16 states | Lilevik: lightning recurrence.  States are float32: 7 flops per
+    # token, channel and state (decay exponent, its exponential, dt x B, multiply-add, multiply-add), at the float32 vector peak
+    C, N, Rk = 2 * width, 16, width // 16
+    xz, xc, dt, bc = r(T, 2 * C + 2 * ff), r(T, C), torch.randn(T, C, device=dev), r(T, Rk + 2 * N)
+    A, bias, Dv = -torch.rand(C, N, device=dev) - 0.1, torch.randn(C, device=dev) - 3, torch.randn(C, device=dev)
+    state = torch.zeros(max(nseq, B), C, N, device=dev)
+    out = r(T, C + ff)
+    scan = lambda n, c: hy_ops.selective_scan(xc[:n], dt[:n], bias, bc[:n], Rk, Rk + N, A, Dv, xz[:n, C:2 * C], state, c, out=out[:n, :C])  # noqa: E731
+    add("hm_selective_scan prefill (%dx%d, %d channels of %d)" % (nseq, seq, C, N), "hm_lightning_recurrence prefill",
+        _event_time(lambda: scan(T, pre), 10), bytes_=T * C * (2 + 4 + 2 + 2) + T * N * 4, flops=T * C * N * 7.0, peak=VALU_F32_TFLOPS)
+    add("hm_selective_scan decode (B=%d)" % B, "hm_lightning_recurrence decode", _event_time(lambda: scan(B, dec)),
+        bytes_=B * C * (N * 8 + 10))
+    w, cb = r(C, 4), r(C)
+    cst = torch.zeros(max(nseq, B), 1, 3, C, device=dev, dtype=bf)
+    add("sm_short_conv + bias + SiLU (T=%d, %d channels)" % (T, C), "hm_delta_gate_norm over all heads",
+        _event_time(lambda: seq_ops.short_conv(xz[:, :C], w, cst, 0, pre, cb, True)), bytes_=T * C * 4)
+    add("sm_short_conv decode (B=%d)" % B, "-", _event_time(lambda: seq_ops.short_conv(xz[:B, :C], w, cst, 0, dec, cb, True)), bytes_=B * C * (4 + 12))
+    prod32, wdt, wx = F32Product(), r(C, Rk), r(Rk + 2 * N, C)
+    add("step-size product, float32 result (T=%d, K=%d)" % (T, Rk), "-", _event_time(lambda: prod32(bc[:, :Rk], wdt)), bytes_=T * C * 4 + T * Rk * 2,
+        flops=2.0 * T * C * Rk)
+    add("d, B, C product (T=%d, K=%d, N=%d)" % (T, C, Rk + 2 * N), "-", _event_time(lambda: torch.nn.functional.linear(xc, wx)), bytes_=T * C * 2,
+        flops=2.0 * T * C * (Rk + 2 * N))
+    LH = width // 128
+    proj = r(T, 4 * LH * 128)
+    decay = torch.rand(LH, device=dev) * 0.1 + 0.9
+    lstate = torch.zeros(max(nseq, B), LH, 128, 128, device=dev)
+    add("hm_lightning_recurrence prefill (%dx%d, %d heads of 128x128)" % (nseq, seq, LH), "-",
+        _event_time(lambda: hy_ops.lightning_recurrence(proj, 0, LH * 128, 2 * LH * 128, LH, 128, 128, decay, lstate, pre), 5),
+        bytes_=T * LH * 128 * (3 * 2 + 4) + nseq * LH * 128 * 128 * 8, flops=T * LH * 4 * 128 * 128, peak=VALU_F32_TFLOPS)
+    projd = proj[:B].contiguous()
+    add("hm_lightning_recurrence decode (B=%d)" % B, "-",
+        _event_time(lambda: hy_ops.lightning_recurrence(projd, 0, LH * 128, 2 * LH * 128, LH, 128, 128, decay, lstate, dec)),
+        bytes_=B * LH * 128 * 128 * 8)
+    o, gcol, ow = torch.randn(T, LH, 128, device=dev), r(T, LH * 128), r(LH * 128)
+    add("hm_delta_gate_norm over all heads (T=%d)" % T, "-",
+        _event_time(lambda: hy_ops.delta_gate_norm(o.view(T, 1, LH * 128), gcol, ow, 1e-5, bf)), bytes_=T * LH * 128 * (4 + 2 + 2))
+    # ---- latent side: stretched rotation, sinks, a reader | Lilevik: plain
+    Q = 3 * rank
+    cache = r(nblk, bs, rank)
+    first, lw = r(T, Q + rank), r(R)
+    q2, qa = r(T, heads * (D + Rd)), r(T, heads, rank)
+    rf, mag = hy_ops.rotary_table(64, 1e4, dev, dict(factor=4.0, original=2048, fast=32.0, slow=1.0))
+    sink = torch.randn(heads, device=dev)
+    add("sm_latent_rope_store stretched (T=%d, H=%d)" % (T, heads), "sm_latent_rope_store",
+        _event_time(lambda: seq_ops.latent_rope_store(first[:, Q:], lw, 1e-5, q2, qa, rf, Rd, heads, D, R, Rd, cache, pre, mag)),
+        bytes_=T * (rank * 4 + heads * Rd * 4))
+    add("sm_latent_rope_store reader (T=%d, H=%d)" % (T, heads), "sm_latent_rope_store",
+        _event_time(lambda: seq_ops.latent_rope_store(None, None, 1e-5, q2, qa, rf, Rd, heads, D, R, Rd, None, pre, mag)),
+        bytes_=T * heads * Rd * 4)
+    add("sm_latent_rope_store (T=%d, H=%d)" % (T, heads), "-",
+        _event_time(lambda: seq_ops.latent_rope_store(first[:, Q:], lw, 1e-5, q2, qa, rf, Rd, heads, D, R, Rd, cache, pre)),
+        bytes_=T * (rank * 4 + heads * Rd * 4))
+    pairs = nseq * seq * (seq + 1) / 2 * heads
+    for name, s in (("+ sink", sink), ("", None)):
+        add("sm_latent_attn_tiles %s, row %d+%d (%dx%d, H=%d)" % (name, R, Rd, nseq, seq, heads), "sm_latent_attn_tiles" if name else "-",
+            _event_time(lambda: seq_ops.latent_attention(qa, cache, pre, 0.07, value_cols=R, sink=s), 5), flops=pairs * 2 * (rank + R))
+    qad = r(B, heads, rank)
+    for name, s in (("+ sink", sink), ("", None)):
+        add("sm_latent_attn_decode %s, row %d+%d (B=%d, ctx=%d)" % (name, R, Rd, B, ctx), "sm_latent_attn_decode" if name else "-",
+            _event_time(lambda: seq_ops.latent_attention(qad, cache, dec, 0.07, value_cols=R, sink=s)), bytes_=B * ctx * rank * 2)
+    # ---- feed-forward: tanh-GELU gate, squared ReLU with a row scale | the clamped GLU
+    gu, zs = xz[:, 2 * C:], xz[:, 2 * C:2 * C + F]
+    sg = torch.rand(T, device=dev)
+    add("sm_gated_act tanh-GELU (T=%d, ff=%d)" % (T, ff), "sm_gated_act clamped", _event_time(
+        lambda: seq_ops.gated_act(gu, seq_ops.ACT_GELU_TANH_GLU, out=out[:, C:])), bytes_=T * ff * 6)
+    add("sm_gated_act clamped (T=%d, ff=%d)" % (T, ff), "-", _event_time(
+        lambda: seq_ops.gated_act(gu, seq_ops.ACT_CLAMPED_GLU, 7.0, 1.702, out=out[:, C:])), bytes_=T * ff * 6)
+    add("hm_relu_squared + row scale (T=%d, ff=%d)" % (T, F), "sm_gated_act clamped",
+        _event_time(lambda: hy_ops.relu_squared(zs, sg, out=out[:, C:C + F])), bytes_=T * F * 4)
+    # ---- router and experts: sigmoid scores + the shared expert's gate, squared-ReLU experts weighted at their input | Lilevik
+    h = r(T, width)
+    rw, rb, gw = torch.randn(E, width, device=dev), torch.randn(E, device=dev) * 0.1, torch.randn(width, device=dev)
+    route = lambda v: seq_ops.moe_route(v, rw, top, score=seq_ops.ROUTE_SIGMOID, renorm=False, gate_w=gw)  # noqa: E731
+    add("sm_moe_route sigmoid + gate (T=%d, E=%d)" % (T, E), "sm_moe_route softmax + bias", _event_time(lambda: route(h)), bytes_=T * width * 2)
+    add("sm_moe_route softmax + bias (T=%d, E=%d)" % (T, E), "-", _event_time(lambda: seq_ops.moe_route(h, rw, top, bias=rb)), bytes_=T * width * 2)
+    idx, wts, _ = route(h)
+    w_up, w_gu, w_down = r(E, F, width), r(E, 2 * F, width), r(E, width, F)
+    t_up = (seq_ops.tile_expert_weights(w_up, 1), seq_ops.tile_expert_weights(w_down))
+    t_glu = (seq_ops.tile_expert_weights(w_gu, 2), t_up[1])
+    inf = float("inf")
+    relu = lambda v, i, w_, form: seq_ops.moe_experts(v, i, w_, w_up, w_down, 0.0, form=form, tiled=t_up, act_kind=seq_ops.ACT_RELU_SQ,  # noqa: E731
+                                                      weight_in=True, combine=False)
+    silu = lambda v, i, w_, form: seq_ops.moe_experts(v, i, w_, w_gu, w_down, inf, 1.0, form=form, tiled=t_glu, act_kind=seq_ops.ACT_SILU_GLU)  # noqa: E731
+    add("sm_moe_tiles128 squared-ReLU experts (T=%d, top %d of %d, F=%d)" % (T, top, E, F), "sm_moe_tiles128 SiLU-gated experts",
+        _event_time(lambda: relu(h, idx, wts, "tiles128"), 5), flops=T * top * 4 * width * F)
+    add("sm_moe_tiles128 SiLU-gated experts (T=%d)" % T, "-", _event_time(lambda: silu(h, idx, wts, "tiles128"), 5), flops=T * top * 6 * width * F)
+    hd = h[:B].contiguous()
+    idx_d, wts_d, _ = route(hd)
+    touched = len(torch.unique(idx_d))
+    add("sm_moe_grouped squared-ReLU experts (T=%d: decode)" % B, "sm_moe_grouped SiLU-gated experts",
+        _event_time(lambda: relu(hd, idx_d, wts_d, "grouped")), bytes_=touched * 2 * F * width * 2)
+    add("sm_moe_grouped SiLU-gated experts (T=%d: decode)" % B, "-", _event_time(lambda: silu(hd, idx_d, wts_d, "grouped")),
+        bytes_=touched * 3 * F * width * 2)
+    # ---- the merged products of a parallel block (vendor GEMMs): first (scan rows + dense gate and up), last (channels + ff)
+    wf, wl, av = r(2 * C + 2 * ff, width), r(width, C + ff), out
+    add("merged first product (T=%d, N=%d, K=%d)" % (T, 2 * C + 2 * ff, width), "-", _event_time(lambda: torch.nn.functional.linear(h, wf), 5),
+        flops=2.0 * T * width * (2 * C + 2 * ff))
+    add("merged last product (T=%d, N=%d, K=%d)" % (T, width, C + ff), "-", _event_time(lambda: torch.nn.functional.linear(av, wl), 5),
+        flops=2.0 * T * width * (C + ff))
+    return rows
+
+
 def main(sizes=("w1024", "w2048"), kernels=True, family="pasizen"):
     out = dict(metric="family comparison", dtype="bf16", data="synthetic (random weights)", throughput=[], kernels=[])
-    beside = {"galupel": ("pasizen", "qwen3"), "lilevik": ("galupel", "lipelix", "qwen3")}.get(family, ("qwen3",))
+    beside = {"galupel": ("pasizen", "qwen3"), "lilevik": ("galupel", "lipelix", "qwen3"), "tafopel": ("lilevik", "qwen3")}.get(family, ("qwen3",))
     for size in sizes:
         for fam in (family,) + beside:
             out["throughput"].append(engine_throughput(fam, size))
     if kernels:
-        out["kernels"] = {"pasizen": kernel_table, "galupel": galupel_kernel_table, "lilevik": lilevik_kernel_table}.get(
+        out["kernels"] = {"pasizen": kernel_table, "galupel": galupel_kernel_table, "lilevik": lilevik_kernel_table,
+                          "tafopel": tafopel_kernel_table}.get(
             family, hymix_kernel_table)()
     return out
