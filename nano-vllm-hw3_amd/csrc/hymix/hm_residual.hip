@@ -104,15 +104,24 @@ __global__ void token_shift_kernel(const T* __restrict__ h, const T* __restrict_
     }
 }
 
-template <typename T>
+// VEC consecutive columns per thread (VEC = 8 where rows allow)
+template <typename T, int VEC>
 __global__ void relu_squared_kernel(const T* __restrict__ z, int64_t z_stride, const float* __restrict__ row_scale,
-                                    T* __restrict__ out, int64_t out_stride, int F) {
-    const int64_t t = blockIdx.x;
+                                    T* __restrict__ out, int64_t out_stride, int64_t n, int F) {
+    const int64_t i = ((int64_t)blockIdx.x * blockDim.x + threadIdx.x) * VEC;
+    if (i >= n) return;
+    struct alignas(sizeof(T) * VEC) Pack { T v[VEC]; };
+    const int64_t t = i / F;
+    const int c = (int)(i - t * F);
     const float rs = row_scale ? row_scale[t] : 1.f;
-    for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < F; c += gridDim.y * blockDim.x) {
-        const float v = fmaxf(to_f(z[(size_t)t * z_stride + c]), 0.f);
-        out[(size_t)t * out_stride + c] = from_f<T>(rs * (v * v));
+    const Pack a = *(const Pack*)(z + (size_t)t * z_stride + c);
+    Pack o;
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) {
+        const float v = fmaxf(to_f(a.v[e]), 0.f);
+        o.v[e] = from_f<T>(rs * (v * v));
     }
+    *(Pack*)(out + (size_t)t * out_stride + c) = o;
 }
 
 }  // namespace hm
@@ -179,10 +188,13 @@ extern "C" int hm_relu_squared(int dtype, const void* z, int64_t z_stride, const
                                int64_t T, int F, void* stream) {
     if (T < 0 || F < 1 || z_stride < F || out_stride < F || (T > 0 && (!z || !out))) { set_error("hm_relu_squared: bad argument"); return HM_EINVAL; }
     if (T == 0) return HM_OK;
-    dim3 grid((unsigned)T, (unsigned)((F + 1023) / 1024));
-    HM_DISPATCH(dtype, "hm_relu_squared",
-                hipLaunchKernelGGL(relu_squared_kernel<DT>, grid, dim3(256), 0, as_stream(stream), (const DT*)z, z_stride,
-                                   row_scale, (DT*)out, out_stride, F));
+    const int64_t n = T * F;
+    const bool wide = F % 8 == 0 && z_stride % 8 == 0 && out_stride % 8 == 0 && ((uintptr_t)z | (uintptr_t)out) % 16 == 0;
+#define HM_RELU2(VEC_)                                                                                                      \
+    hipLaunchKernelGGL((relu_squared_kernel<DT, VEC_>), dim3((unsigned)((n / VEC_ + 255) / 256)), dim3(256), 0, as_stream(stream), \
+                       (const DT*)z, z_stride, row_scale, (DT*)out, out_stride, n, F)
+    HM_DISPATCH(dtype, "hm_relu_squared", if (wide) HM_RELU2(8); else HM_RELU2(1));
+#undef HM_RELU2
     HM_CHECK_LAUNCH("hm_relu_squared");
     return HM_OK;
 }

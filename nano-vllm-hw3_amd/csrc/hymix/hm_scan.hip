@@ -22,14 +22,27 @@ __device__ __forceinline__ float group_sum(float v) {
     return v;
 }
 
-__device__ __forceinline__ float softplus_f(float v) { return fmaxf(v, 0.f) + log1pf(__expf(-fabsf(v))); }
+// ln(1 + e^v) = max(v, 0) + ln(1 + u), u = e^-|v|: the logarithm of the rounded sum loses small u, whose first series terms
+// then serve instead (u < 1/16: the next one is below 2^-26 of the sum)
+__device__ __forceinline__ float softplus_f(float v) {
+    const float u = __builtin_amdgcn_exp2f(-fabsf(v) * 1.4426950408889634f);
+    const float lg = __builtin_amdgcn_logf(1.f + u) * 0.69314718055994531f;
+    const float ps = u * (1.f - u * (0.5f - u * (0.33333333f - u * (0.25f - u * (0.2f - u * 0.16666667f)))));
+    return fmaxf(v, 0.f) + (u < 0.0625f ? ps : lg);
+}
+
+// z sigmoid(z) from the hardware's exponential and reciprocal (float32, a few units in the last place)
+__device__ __forceinline__ float silu_f(float z) { return z * __builtin_amdgcn_rcpf(1.f + __expf(-z)); }
+
+// tokens staged at a time: as many as keep the pairs and the B, C rows of a chunk in a few tens of KB
+constexpr int scan_chunk(int L, int NP) { return L <= 2 ? 16 : (NP <= 64 ? 32 : (NP <= 256 ? 16 : 8)); }
 
 // A workgroup of 256 threads owns 256 / L channels of one sequence; a channel's states are spread over L neighbouring lanes,
 // NS in each lane's registers (L * NS >= N; the lanes beyond N hold zeros that meet zero B and C).  CH tokens are staged at
-// a time: every (token, channel) is fetched by one thread, which turns it into the pair (dt, dt x) in LDS; B and C of the
-// tokens lie beside them.  The next chunk is requested from global memory before the current one runs.  A channel's sum over
-// the states replaces its pair in LDS, and the thread that fetched the element adds the skip, applies the gate and stores.
-template <typename T, int L, int NS, int CH>
+// a time: a thread fetches VEC neighbouring channels of a token and turns them into pairs (dt, dt x) in LDS, B and C of the
+// tokens lie beside them.  The next chunk is requested from global memory before the current one runs.  A channel's sums over
+// the states are kept by its lanes in turn (lane t % L keeps token t's) and go to LDS L tokens at a time; the thread that fetched a token's channels adds the skip, applies the gate and stores.
+template <typename T, int L, int NS, int CH, int VEC>
 __global__ __launch_bounds__(256) void selective_scan_kernel(const T* __restrict__ x, int64_t x_stride,
                                                              const float* __restrict__ dt_pre, int64_t dt_stride,
                                                              const float* __restrict__ dt_bias, const T* __restrict__ bc,
@@ -39,10 +52,17 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(const T* __restrict
                                                              const int32_t* __restrict__ qstart,
                                                              const int32_t* __restrict__ seq_pos0,
                                                              const int32_t* __restrict__ seq_slot, T* __restrict__ out,
-                                                             int64_t out_stride, int C, int N) {
-    constexpr int CPW = 256 / L, NP = L * NS, EL = CH * CPW, NR = (EL + 255) / 256, BC = CH * 2 * NP, NB = (BC + 255) / 256;
-    __shared__ __attribute__((aligned(16))) float2 step_lds[EL];            // (dt, dt x); then the sum over the states in .x
-    __shared__ __attribute__((aligned(16))) float bc_lds[BC];               // per token B[NP], C[NP]
+                                                             int64_t out_stride, int C, int N, int whole) {
+    struct alignas(sizeof(T) * VEC) Pack { T v[VEC]; };
+    struct alignas(4 * VEC) PackF { float v[VEC]; };
+    typedef float StV __attribute__((ext_vector_type(NS)));
+    constexpr int CPW = 256 / L, NP = L * NS, Q = CPW / VEC, ROWS = 256 / Q;       // ROWS tokens are fetched at a time
+    constexpr int UN = L >= 4 ? 1 : 4 / L;     // groups of L tokens per round of the loop: four tokens at least
+    constexpr int NR = (CH + ROWS - 1) / ROWS, BC = CH * 2 * NP, NB = (BC + 255) / 256;
+    // (one token more than a chunk: the walk reads ahead)
+    __shared__ __attribute__((aligned(16))) float2 step_lds[(CH + 1) * CPW];      // (dt, dt x)
+    __shared__ __attribute__((aligned(16))) float bc_lds[BC + 2 * NP];            // per token B[NP], C[NP]
+    __shared__ __attribute__((aligned(16))) float y_lds[CH * CPW];                // the sums over the states
     const int b = blockIdx.x;
     const int q0 = qstart[b], n = qstart[b + 1] - q0;
     if (n <= 0) return;
@@ -51,31 +71,50 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(const T* __restrict
     float* st = state + ((size_t)seq_slot[b] * C + ch) * N + n0;
     const bool fresh = seq_pos0[b] == 0;
     float s[NS], a2[NS];
+    if (whole) {                               // N == NP and 16-byte rows: a lane's states in whole vectors
+        StV sv = {}, av = {};
+        if (ch < C) {
+            if (!fresh) sv = *(const StV*)st;
+            av = *(const StV*)(A + (size_t)ch * N + n0);
+        }
 #pragma unroll
-    for (int i = 0; i < NS; ++i) {
-        const bool in = ch < C && n0 + i < N;
-        s[i] = in && !fresh ? st[i] : 0.f;
-        a2[i] = in ? A[(size_t)ch * N + n0 + i] * 1.4426950408889634f : 0.f;
-    }
-    // the elements this thread fetches and finishes: token el_t of the chunk, channel el_c
-    float el_bias[NR], el_D[NR];
+        for (int i = 0; i < NS; ++i) { s[i] = sv[i]; a2[i] = av[i] * 1.4426950408889634f; }
+    } else {
 #pragma unroll
-    for (int k = 0; k < NR; ++k) {
-        const int e = tid + 256 * k, c = c0 + e % CPW;
-        el_bias[k] = e < EL && c < C ? dt_bias[c] : 0.f;
-        el_D[k] = e < EL && c < C ? D[c] : 0.f;
+        for (int i = 0; i < NS; ++i) {
+            const bool in = ch < C && n0 + i < N;
+            s[i] = in && !fresh ? st[i] : 0.f;
+            a2[i] = in ? A[(size_t)ch * N + n0 + i] * 1.4426950408889634f : 0.f;
+        }
     }
-    T rx[NR], rz[NR], rbc[NB];
-    float rdt[NR];
+    // what this thread fetches and finishes: channels cq .. cq + VEC of the tokens row0, row0 + ROWS, ... of a chunk
+    const int row0 = tid / Q, cl = tid % Q * VEC, cq = c0 + cl;
+    const bool mine = cq < C;                  // (VEC divides C)
+    float bias[VEC], skip[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) {
+        bias[e] = mine ? dt_bias[cq + e] : 0.f;
+        skip[e] = mine ? D[cq + e] : 0.f;
+    }
+    const T* px = x + (size_t)(q0 + row0) * x_stride + cq;
+    const T* pz = z + (size_t)(q0 + row0) * z_stride + cq;
+    const float* pd = dt_pre + (size_t)(q0 + row0) * dt_stride + cq;
+    T* po = out + (size_t)(q0 + row0) * out_stride + cq;
+    Pack rx[NR], rz[NR];
+    PackF rd[NR];
+    T rbc[NB];
     auto request = [&](int tok0) {
 #pragma unroll
         for (int k = 0; k < NR; ++k) {
-            const int e = tid + 256 * k, tok = tok0 + e / CPW, c = c0 + e % CPW;
-            const bool in = e < EL && tok < n && c < C;
-            const size_t row = (size_t)(q0 + tok);
-            rx[k] = in ? x[row * x_stride + c] : from_f<T>(0.f);
-            rz[k] = in ? z[row * z_stride + c] : from_f<T>(0.f);
-            rdt[k] = in ? dt_pre[row * dt_stride + c] : 0.f;
+            const int t = row0 + k * ROWS;
+            const bool in = mine && t < CH && tok0 + t < n;
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) { rx[k].v[e] = rz[k].v[e] = from_f<T>(0.f); rd[k].v[e] = 0.f; }
+            if (in) {
+                rx[k] = *(const Pack*)(px + (int64_t)(tok0 + k * ROWS) * x_stride);
+                rz[k] = *(const Pack*)(pz + (int64_t)(tok0 + k * ROWS) * z_stride);
+                rd[k] = *(const PackF*)(pd + (int64_t)(tok0 + k * ROWS) * dt_stride);
+            }
         }
 #pragma unroll
         for (int k = 0; k < NB; ++k) {
@@ -86,14 +125,19 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(const T* __restrict
     };
     request(0);
     for (int tok0 = 0; tok0 < n; tok0 += CH) {
-        float xs[NR], zs[NR];
+        Pack cx[NR], cz[NR];
 #pragma unroll
         for (int k = 0; k < NR; ++k) {
-            const int e = tid + 256 * k;
-            xs[k] = to_f(rx[k]);
-            zs[k] = to_f(rz[k]);
-            const float dt = softplus_f(rdt[k] + el_bias[k]);
-            if (e < EL) step_lds[e] = make_float2(dt, dt * xs[k]);
+            const int t = row0 + k * ROWS;
+            cx[k] = rx[k];
+            cz[k] = rz[k];
+            if (t < CH) {
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) {
+                    const float dt = softplus_f(rd[k].v[e] + bias[e]);
+                    step_lds[t * CPW + cl + e] = make_float2(dt, dt * to_f(cx[k].v[e]));
+                }
+            }
         }
 #pragma unroll
         for (int k = 0; k < NB; ++k) {
@@ -102,39 +146,77 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(const T* __restrict
         }
         __syncthreads();
         if (tok0 + CH < n) request(tok0 + CH);
-        auto step = [&](int t) {
-            const float2 d = step_lds[t * CPW + chl];
+        struct Token { float2 d; float b[NS], c[NS]; };
+        auto fetch = [&](int t) {
+            Token w;
             const float* pb = bc_lds + t * 2 * NP + n0;
+            w.d = step_lds[t * CPW + chl];
+#pragma unroll
+            for (int i = 0; i < NS; ++i) { w.b[i] = pb[i]; w.c[i] = pb[NP + i]; }
+            return w;
+        };
+        auto step = [&](const Token& w) {
             float acc = 0.f;
 #pragma unroll
             for (int i = 0; i < NS; ++i) {
-                s[i] = __builtin_amdgcn_exp2f(d.x * a2[i]) * s[i] + d.y * pb[i];
-                acc += s[i] * pb[NP + i];
+                s[i] = __builtin_amdgcn_exp2f(w.d.x * a2[i]) * s[i] + w.d.y * w.b[i];
+                acc += s[i] * w.c[i];
             }
-            acc = group_sum<L>(acc);
-            if (slice == 0) step_lds[t * CPW + chl].x = acc;       // (only this group of lanes reads the pair)
+            return group_sum<L>(acc);
         };
         const int nt = min(CH, n - tok0);
-        if (CH > 1 && nt == CH) {
-#pragma unroll 4
-            for (int t = 0; t < CH; ++t) step(t);
-        } else {
-            for (int t = 0; t < nt; ++t) step(t);
+        int t = 0;
+        Token cur = fetch(0);
+        if (CH >= L) {
+#pragma unroll 1
+            for (; t + L * UN <= nt; t += L * UN) {
+#pragma unroll
+                for (int u = 0; u < UN; ++u) {
+                    float keep = 0.f;
+#pragma unroll
+                    for (int j = 0; j < L; ++j) {
+                        const Token nxt = fetch(t + u * L + j + 1);
+                        const float v = step(cur);
+                        keep = slice == j ? v : keep;
+                        cur = nxt;
+                    }
+                    y_lds[(t + u * L + slice) * CPW + chl] = keep;
+                }
+            }
+        }
+        for (; t < nt; ++t) {
+            const Token nxt = fetch(t + 1);
+            const float v = step(cur);
+            cur = nxt;
+            if (slice == 0) y_lds[t * CPW + chl] = v;
         }
         __syncthreads();
 #pragma unroll
         for (int k = 0; k < NR; ++k) {
-            const int e = tid + 256 * k, tok = tok0 + e / CPW, c = c0 + e % CPW;
-            if (e < EL && tok < n && c < C) {
-                const float y = step_lds[e].x + el_D[k] * xs[k];
-                out[(size_t)(q0 + tok) * out_stride + c] = from_f<T>(y * zs[k] / (1.f + __expf(-zs[k])));
+            const int tr = row0 + k * ROWS;
+            if (mine && tr < nt) {
+                Pack o;
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) {
+                    const float y = y_lds[tr * CPW + cl + e] + skip[e] * to_f(cx[k].v[e]);
+                    o.v[e] = from_f<T>(y * silu_f(to_f(cz[k].v[e])));
+                }
+                *(Pack*)(po + (int64_t)(tok0 + k * ROWS) * out_stride) = o;
             }
         }
-        // (the next deposit writes elements that this thread alone has just read; B and C were last read before the barrier)
+        // (what the next deposit overwrites was last read before the barrier; the sums are replaced behind the next one)
     }
+    if (ch >= C) return;
+    if (whole) {
+        StV sv;
 #pragma unroll
-    for (int i = 0; i < NS; ++i)
-        if (ch < C && n0 + i < N) st[i] = s[i];
+        for (int i = 0; i < NS; ++i) sv[i] = s[i];
+        *(StV*)st = sv;
+    } else {
+#pragma unroll
+        for (int i = 0; i < NS; ++i)
+            if (n0 + i < N) st[i] = s[i];
+    }
 }
 
 template <typename DT>
@@ -142,18 +224,30 @@ static void launch_scan(const void* x, int64_t x_stride, const float* dt_pre, in
                         int64_t bc_stride, int b_off, int c_off, const float* A, const float* D, const void* z, int64_t z_stride,
                         float* state, const int32_t* qstart, const int32_t* seq_pos0, const int32_t* seq_slot, void* out,
                         int64_t out_stride, int B, int C, int N, int max_q, hipStream_t s) {
-#define HM_SCAN(L, NS, CH)                                                                                                   \
-    hipLaunchKernelGGL((selective_scan_kernel<DT, L, NS, CH>), dim3((unsigned)B, (unsigned)((C + 256 / L - 1) / (256 / L))), dim3(256), \
-                       0, s, (const DT*)x, x_stride, dt_pre, dt_stride, dt_bias, (const DT*)bc, bc_stride, b_off, c_off, A, D,  \
-                       (const DT*)z, z_stride, state, qstart, seq_pos0, seq_slot, (DT*)out, out_stride, C, N)
-#define HM_SCAN_T(L, NS) do { if (max_q <= 1) HM_SCAN(L, NS, 1); else HM_SCAN(L, NS, 16); } while (0)
-    // states per lane: more of them share a token's fetches and sums, fewer give more lanes to a small batch
+    // whole vectors of states; packs of four channels where every row starts on one
+    const bool st16 = N % 4 == 0 && ((uintptr_t)state | (uintptr_t)A) % 16 == 0;
+    const int64_t strides = C | x_stride | dt_stride | z_stride | out_stride;
+    const bool wide = strides % 4 == 0 && ((uintptr_t)x | (uintptr_t)dt_pre | (uintptr_t)z | (uintptr_t)out) % 16 == 0;
+#define HM_SCAN(L, NS, CH, VEC)                                                                                              \
+    hipLaunchKernelGGL((selective_scan_kernel<DT, L, NS, CH, VEC>), dim3((unsigned)B, (unsigned)((C + 256 / L - 1) / (256 / L))), \
+                       dim3(256), 0, s, (const DT*)x, x_stride, dt_pre, dt_stride, dt_bias, (const DT*)bc, bc_stride, b_off, c_off, \
+                       A, D, (const DT*)z, z_stride, state, qstart, seq_pos0, seq_slot, (DT*)out, out_stride, C, N,           \
+                       st16 && N == L * NS)
+#define HM_SCAN_V(L, NS, CH) do { if (wide) HM_SCAN(L, NS, CH, 4); else HM_SCAN(L, NS, CH, 1); } while (0)
+#define HM_SCAN_T(L, NS)                                                                 \
+    do {                                                                                 \
+        if (NS == 8 && max_q <= 1) HM_SCAN_V(L, NS, (NS == 8 ? 1 : scan_chunk(L, L * NS))); \
+        else HM_SCAN_V(L, NS, scan_chunk(L, L * NS));                                    \
+    } while (0)
+    // states per lane: more of them share a token's fetches and sums, fewer give more lanes to a small batch; a single token is
+    // bound by its state's traffic and takes the longest vectors
     const int64_t states = (int64_t)B * C * N;
-    const int ns = N > 8 && N <= 128 && states < 8 * 48 * 1024 ? (N <= 32 && states < 4 * 48 * 1024 ? 2 : 4) : 8;
+    const int ns = max_q <= 1 || N > 128 ? 8 : (N <= 32 ? (states < 288 * 1024 ? 2 : 4) : (states < 512 * 1024 ? 4 : 8));
     if (ns == 2) {
-        if (N <= 16) HM_SCAN_T(8, 2); else HM_SCAN_T(16, 2);
+        if (N <= 8) HM_SCAN_T(4, 2); else if (N <= 16) HM_SCAN_T(8, 2); else HM_SCAN_T(16, 2);
     } else if (ns == 4) {
-        if (N <= 16) HM_SCAN_T(4, 4); else if (N <= 32) HM_SCAN_T(8, 4); else if (N <= 64) HM_SCAN_T(16, 4); else HM_SCAN_T(32, 4);
+        if (N <= 8) HM_SCAN_T(2, 4); else if (N <= 16) HM_SCAN_T(4, 4); else if (N <= 32) HM_SCAN_T(8, 4);
+        else if (N <= 64) HM_SCAN_T(16, 4); else HM_SCAN_T(32, 4);
     } else if (N <= 8) HM_SCAN_T(1, 8);
     else if (N <= 16) HM_SCAN_T(2, 8);
     else if (N <= 32) HM_SCAN_T(4, 8);
@@ -162,6 +256,7 @@ static void launch_scan(const void* x, int64_t x_stride, const float* dt_pre, in
     else if (N <= 256) HM_SCAN_T(32, 8);
     else HM_SCAN_T(64, 8);
 #undef HM_SCAN_T
+#undef HM_SCAN_V
 #undef HM_SCAN
 }
 

@@ -25,12 +25,26 @@ __global__ __launch_bounds__(64) void short_conv_kernel(const T* __restrict__ x,
     T* st = state + ((size_t)seq_slot[b] * runs + run) * (size_t)(taps - 1) * W + c;      // (taps == 1: not touched)
     const T* xc = x + (size_t)q0 * row_stride + c;
     float wr[TAPS][VEC], hist[TAPS][VEC], bs[VEC];
+    if (VEC > 1 && taps == TAPS) {                  // the thread's weights are VEC * TAPS neighbours: whole packs
+        Pack wp[TAPS];
 #pragma unroll
-    for (int j = 0; j < TAPS; ++j)
+        for (int k = 0; k < TAPS; ++k) wp[k] = *(const Pack*)(w + (size_t)c * TAPS + k * VEC);
 #pragma unroll
-        for (int e = 0; e < VEC; ++e) wr[j][e] = j >= skip ? to_f(w[(size_t)(c + e) * taps + j - skip]) : 0.f;
+        for (int j = 0; j < TAPS; ++j)
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) bs[e] = bias ? to_f(bias[c + e]) : 0.f;
+            for (int e = 0; e < VEC; ++e) wr[j][e] = to_f(wp[(e * TAPS + j) / VEC].v[(e * TAPS + j) % VEC]);
+    } else {
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) wr[j][e] = j >= skip ? to_f(w[(size_t)(c + e) * taps + j - skip]) : 0.f;
+    }
+    Pack bp;
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) bp.v[e] = from_f<T>(0.f);
+    if (bias != nullptr) bp = *(const Pack*)(bias + c);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) bs[e] = to_f(bp.v[e]);
     // hist[j] = the input TAPS - 1 - j tokens before the current one: rows of this step, then the carried inputs (state row
     // k = the input taps-1-k tokens before the portion), zero before the sequence's start whatever the slot holds
 #pragma unroll
@@ -44,8 +58,8 @@ __global__ __launch_bounds__(64) void short_conv_kernel(const T* __restrict__ x,
         for (int e = 0; e < VEC; ++e) hist[j][e] = to_f(v.v[e]);
     }
     const int nt = min(kChunk, n - t0);
-    auto step = [&](int i) {
-        const Pack cur = *(const Pack*)(xc + (size_t)(t0 + i) * row_stride);
+    auto row = [&](int i) { return *(const Pack*)(xc + (size_t)(t0 + i) * row_stride); };
+    auto step = [&](int i, const Pack& cur) {
         Pack o;
 #pragma unroll
         for (int e = 0; e < VEC; ++e) {
@@ -53,7 +67,7 @@ __global__ __launch_bounds__(64) void short_conv_kernel(const T* __restrict__ x,
             float acc = bs[e] + wr[TAPS - 1][e] * v;
 #pragma unroll
             for (int j = 0; j < TAPS - 1; ++j) acc += wr[j][e] * hist[j][e];
-            if (silu) acc = acc / (1.f + __expf(-acc));
+            if (silu) acc = acc * __builtin_amdgcn_rcpf(1.f + __expf(-acc));
             o.v[e] = from_f<T>(add_input ? v + acc : acc);
 #pragma unroll
             for (int j = 0; j + 1 < TAPS - 1; ++j) hist[j][e] = hist[j + 1][e];
@@ -62,10 +76,17 @@ __global__ __launch_bounds__(64) void short_conv_kernel(const T* __restrict__ x,
         *(Pack*)(out + (size_t)(q0 + t0 + i) * W + c) = o;
     };
     if (nt == kChunk) {
-#pragma unroll 4
-        for (int i = 0; i < kChunk; ++i) step(i);
+        constexpr int AHEAD = VEC > 1 ? 8 : 4;      // rows requested together
+#pragma unroll 1
+        for (int i = 0; i < kChunk; i += AHEAD) {
+            Pack cur[AHEAD];
+#pragma unroll
+            for (int k = 0; k < AHEAD; ++k) cur[k] = row(i + k);
+#pragma unroll
+            for (int k = 0; k < AHEAD; ++k) step(i + k, cur[k]);
+        }
     } else {
-        for (int i = 0; i < nt; ++i) step(i);
+        for (int i = 0; i < nt; ++i) step(i, row(i));
     }
     if (blockIdx.x != 0 || taps == 1) return;
     for (int k = 0; k < taps - 1; ++k) {           // ascending: a row is read (k + n > k) before it is replaced
@@ -105,7 +126,7 @@ extern "C" int sm_short_conv(int dtype, const void* x, int64_t row_stride, const
     }
     if (B == 0 || max_q == 0) return SM_OK;
     const int full = dtype == SM_BF16 ? 8 : 4;     // 16-byte packs where every row and the state rows start on one
-    const bool wide = W % full == 0 && row_stride % full == 0 && ((uintptr_t)x | (uintptr_t)state | (uintptr_t)out) % 16 == 0;
+    const bool wide = W % full == 0 && row_stride % full == 0 && ((uintptr_t)x | (uintptr_t)w | (uintptr_t)bias | (uintptr_t)state | (uintptr_t)out) % 16 == 0;
     const int vec = wide ? full : 1;
     const dim3 grid((unsigned)((max_q + kChunk - 1) / kChunk), (unsigned)((W + 64 * vec - 1) / (64 * vec)), (unsigned)B);
 #define SM_CONV_ARGS grid, as_stream(stream), x, row_stride, w, bias, silu, add_input, state, run, runs, qstart, seq_pos0, seq_slot, out, W, taps

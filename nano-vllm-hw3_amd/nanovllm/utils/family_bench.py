@@ -203,6 +203,18 @@ def _event_time(fn, reps=20):
     return a.elapsed_time(b) * 1e-3 / reps
 
 
+def _graph_time(fn, reps=20):
+    """Seconds per launch from a replayed hipGraph: what a kernel of a few microseconds takes without the host's share (for
+    this package's own kernels; vendor products are timed by events)."""
+    fn()
+    torch.cuda.synchronize()
+    g = torch.cuda.CUDAGraph()
+    with torch.cuda.graph(g):
+        for _ in range(reps):
+            fn()
+    return _event_time(g.replay, 3) / reps
+
+
 def kernel_table(width=2048, heads=16, rank=256, ff=6144, T=8192, seq=1024, B=64, ctx=1024, streams=4, taps=4):
     """Seconds per launch of every libseqmix kernel at a layer's size, the bound it works against (bytes / HBM peak or
     flops / matrix peak) and the fraction of that bound it reaches; beside each the like kernel of the Qwen3 path."""
@@ -773,15 +785,15 @@ def tafopel_kernel_table(width=2048, heads=16, rank=256, ff=6144, T=8192, seq=10
     nblk = max(nblk_p, nblk_d)
     # ---- residual boundary: add + layer norm, with and without the experts' rows | Lilevik: tanh norms
     x, y, nw = torch.randn(T, width, device=dev), r(T, width), r(width)
-    add("hm_layer_norm_residual (T=%d)" % T, "hm_dyt_residual", _event_time(lambda: hy_ops.layer_norm_residual(x, y, nw, 1e-5, bf)),
+    add("hm_layer_norm_residual (T=%d)" % T, "hm_dyt_residual", _graph_time(lambda: hy_ops.layer_norm_residual(x, y, nw, 1e-5, bf)),
         bytes_=T * width * (8 + 2 + 2))
     top, E, F = 4, 16, ff // 4
     prod = r(T * top + 128 * E, width)
     pair_row = torch.randperm(T * top, device=dev).int()
     add("hm_layer_norm_residual + expert rows, top %d (T=%d)" % (top, T), "sm_moe_combine + hm_dyt_residual",
-        _event_time(lambda: hy_ops.layer_norm_residual(x, y, nw, 1e-5, bf, routed=(prod, pair_row, None))), bytes_=T * width * (8 + 2 + 2 + 2 * top))
+        _graph_time(lambda: hy_ops.layer_norm_residual(x, y, nw, 1e-5, bf, routed=(prod, pair_row, None))), bytes_=T * width * (8 + 2 + 2 + 2 * top))
     n1, n2 = (r(width), r(width), torch.rand(1, device=dev)), (r(width), r(width), torch.rand(1, device=dev))
-    add("hm_dyt_residual (T=%d)" % T, "-", _event_time(lambda: hy_ops.dyt_residual(x, y, n1, n2, bf)), bytes_=T * width * (8 + 2 + 2))
+    add("hm_dyt_residual (T=%d)" % T, "-", _graph_time(lambda: hy_ops.dyt_residual(x, y, n1, n2, bf)), bytes_=T * width * (8 + 2 + 2))
     # ---- selective scan: 2 x width channels of 16 states | Lilevik: lightning recurrence.  States are float32: 7 flops per
     # token, channel and state (decay exponent, its exponential, dt x B, multiply-add, multiply-add), at the float32 vector peak
     C, N, Rk = 2 * width, 16, width // 16
@@ -791,14 +803,14 @@ def tafopel_kernel_table(width=2048, heads=16, rank=256, ff=6144, T=8192, seq=10
     out = r(T, C + ff)
     scan = lambda n, c: hy_ops.selective_scan(xc[:n], dt[:n], bias, bc[:n], Rk, Rk + N, A, Dv, xz[:n, C:2 * C], state, c, out=out[:n, :C])  # noqa: E731
     add("hm_selective_scan prefill (%dx%d, %d channels of %d)" % (nseq, seq, C, N), "hm_lightning_recurrence prefill",
-        _event_time(lambda: scan(T, pre), 10), bytes_=T * C * (2 + 4 + 2 + 2) + T * N * 4, flops=T * C * N * 7.0, peak=VALU_F32_TFLOPS)
-    add("hm_selective_scan decode (B=%d)" % B, "hm_lightning_recurrence decode", _event_time(lambda: scan(B, dec)),
+        _graph_time(lambda: scan(T, pre), 10), bytes_=T * C * (2 + 4 + 2 + 2) + T * N * 4, flops=T * C * N * 7.0, peak=VALU_F32_TFLOPS)
+    add("hm_selective_scan decode (B=%d)" % B, "hm_lightning_recurrence decode", _graph_time(lambda: scan(B, dec)),
         bytes_=B * C * (N * 8 + 10))
     w, cb = r(C, 4), r(C)
     cst = torch.zeros(max(nseq, B), 1, 3, C, device=dev, dtype=bf)
     add("sm_short_conv + bias + SiLU (T=%d, %d channels)" % (T, C), "hm_delta_gate_norm over all heads",
-        _event_time(lambda: seq_ops.short_conv(xz[:, :C], w, cst, 0, pre, cb, True)), bytes_=T * C * 4)
-    add("sm_short_conv decode (B=%d)" % B, "-", _event_time(lambda: seq_ops.short_conv(xz[:B, :C], w, cst, 0, dec, cb, True)), bytes_=B * C * (4 + 12))
+        _graph_time(lambda: seq_ops.short_conv(xz[:, :C], w, cst, 0, pre, cb, True)), bytes_=T * C * 4)
+    add("sm_short_conv decode (B=%d)" % B, "-", _graph_time(lambda: seq_ops.short_conv(xz[:B, :C], w, cst, 0, dec, cb, True)), bytes_=B * C * (4 + 12))
     prod32, wdt, wx = F32Product(), r(C, Rk), r(Rk + 2 * N, C)
     add("step-size product, float32 result (T=%d, K=%d)" % (T, Rk), "-", _event_time(lambda: prod32(bc[:, :Rk], wdt)), bytes_=T * C * 4 + T * Rk * 2,
         flops=2.0 * T * C * Rk)
@@ -809,15 +821,15 @@ def tafopel_kernel_table(width=2048, heads=16, rank=256, ff=6144, T=8192, seq=10
     decay = torch.rand(LH, device=dev) * 0.1 + 0.9
     lstate = torch.zeros(max(nseq, B), LH, 128, 128, device=dev)
     add("hm_lightning_recurrence prefill (%dx%d, %d heads of 128x128)" % (nseq, seq, LH), "-",
-        _event_time(lambda: hy_ops.lightning_recurrence(proj, 0, LH * 128, 2 * LH * 128, LH, 128, 128, decay, lstate, pre), 5),
+        _graph_time(lambda: hy_ops.lightning_recurrence(proj, 0, LH * 128, 2 * LH * 128, LH, 128, 128, decay, lstate, pre), 5),
         bytes_=T * LH * 128 * (3 * 2 + 4) + nseq * LH * 128 * 128 * 8, flops=T * LH * 4 * 128 * 128, peak=VALU_F32_TFLOPS)
     projd = proj[:B].contiguous()
     add("hm_lightning_recurrence decode (B=%d)" % B, "-",
-        _event_time(lambda: hy_ops.lightning_recurrence(projd, 0, LH * 128, 2 * LH * 128, LH, 128, 128, decay, lstate, dec)),
+        _graph_time(lambda: hy_ops.lightning_recurrence(projd, 0, LH * 128, 2 * LH * 128, LH, 128, 128, decay, lstate, dec)),
         bytes_=B * LH * 128 * 128 * 8)
     o, gcol, ow = torch.randn(T, LH, 128, device=dev), r(T, LH * 128), r(LH * 128)
     add("hm_delta_gate_norm over all heads (T=%d)" % T, "-",
-        _event_time(lambda: hy_ops.delta_gate_norm(o.view(T, 1, LH * 128), gcol, ow, 1e-5, bf)), bytes_=T * LH * 128 * (4 + 2 + 2))
+        _graph_time(lambda: hy_ops.delta_gate_norm(o.view(T, 1, LH * 128), gcol, ow, 1e-5, bf)), bytes_=T * LH * 128 * (4 + 2 + 2))
     # ---- latent side: stretched rotation, sinks, a reader | Lilevik: plain
     Q = 3 * rank
     cache = r(nblk, bs, rank)
@@ -826,37 +838,37 @@ def tafopel_kernel_table(width=2048, heads=16, rank=256, ff=6144, T=8192, seq=10
     rf, mag = hy_ops.rotary_table(64, 1e4, dev, dict(factor=4.0, original=2048, fast=32.0, slow=1.0))
     sink = torch.randn(heads, device=dev)
     add("sm_latent_rope_store stretched (T=%d, H=%d)" % (T, heads), "sm_latent_rope_store",
-        _event_time(lambda: seq_ops.latent_rope_store(first[:, Q:], lw, 1e-5, q2, qa, rf, Rd, heads, D, R, Rd, cache, pre, mag)),
+        _graph_time(lambda: seq_ops.latent_rope_store(first[:, Q:], lw, 1e-5, q2, qa, rf, Rd, heads, D, R, Rd, cache, pre, mag)),
         bytes_=T * (rank * 4 + heads * Rd * 4))
     add("sm_latent_rope_store reader (T=%d, H=%d)" % (T, heads), "sm_latent_rope_store",
-        _event_time(lambda: seq_ops.latent_rope_store(None, None, 1e-5, q2, qa, rf, Rd, heads, D, R, Rd, None, pre, mag)),
+        _graph_time(lambda: seq_ops.latent_rope_store(None, None, 1e-5, q2, qa, rf, Rd, heads, D, R, Rd, None, pre, mag)),
         bytes_=T * heads * Rd * 4)
     add("sm_latent_rope_store (T=%d, H=%d)" % (T, heads), "-",
-        _event_time(lambda: seq_ops.latent_rope_store(first[:, Q:], lw, 1e-5, q2, qa, rf, Rd, heads, D, R, Rd, cache, pre)),
+        _graph_time(lambda: seq_ops.latent_rope_store(first[:, Q:], lw, 1e-5, q2, qa, rf, Rd, heads, D, R, Rd, cache, pre)),
         bytes_=T * (rank * 4 + heads * Rd * 4))
     pairs = nseq * seq * (seq + 1) / 2 * heads
     for name, s in (("+ sink", sink), ("", None)):
         add("sm_latent_attn_tiles %s, row %d+%d (%dx%d, H=%d)" % (name, R, Rd, nseq, seq, heads), "sm_latent_attn_tiles" if name else "-",
-            _event_time(lambda: seq_ops.latent_attention(qa, cache, pre, 0.07, value_cols=R, sink=s), 5), flops=pairs * 2 * (rank + R))
+            _graph_time(lambda: seq_ops.latent_attention(qa, cache, pre, 0.07, value_cols=R, sink=s), 5), flops=pairs * 2 * (rank + R))
     qad = r(B, heads, rank)
     for name, s in (("+ sink", sink), ("", None)):
         add("sm_latent_attn_decode %s, row %d+%d (B=%d, ctx=%d)" % (name, R, Rd, B, ctx), "sm_latent_attn_decode" if name else "-",
-            _event_time(lambda: seq_ops.latent_attention(qad, cache, dec, 0.07, value_cols=R, sink=s)), bytes_=B * ctx * rank * 2)
+            _graph_time(lambda: seq_ops.latent_attention(qad, cache, dec, 0.07, value_cols=R, sink=s)), bytes_=B * ctx * rank * 2)
     # ---- feed-forward: tanh-GELU gate, squared ReLU with a row scale | the clamped GLU
     gu, zs = xz[:, 2 * C:], xz[:, 2 * C:2 * C + F]
     sg = torch.rand(T, device=dev)
-    add("sm_gated_act tanh-GELU (T=%d, ff=%d)" % (T, ff), "sm_gated_act clamped", _event_time(
+    add("sm_gated_act tanh-GELU (T=%d, ff=%d)" % (T, ff), "sm_gated_act clamped", _graph_time(
         lambda: seq_ops.gated_act(gu, seq_ops.ACT_GELU_TANH_GLU, out=out[:, C:])), bytes_=T * ff * 6)
-    add("sm_gated_act clamped (T=%d, ff=%d)" % (T, ff), "-", _event_time(
+    add("sm_gated_act clamped (T=%d, ff=%d)" % (T, ff), "-", _graph_time(
         lambda: seq_ops.gated_act(gu, seq_ops.ACT_CLAMPED_GLU, 7.0, 1.702, out=out[:, C:])), bytes_=T * ff * 6)
     add("hm_relu_squared + row scale (T=%d, ff=%d)" % (T, F), "sm_gated_act clamped",
-        _event_time(lambda: hy_ops.relu_squared(zs, sg, out=out[:, C:C + F])), bytes_=T * F * 4)
+        _graph_time(lambda: hy_ops.relu_squared(zs, sg, out=out[:, C:C + F])), bytes_=T * F * 4)
     # ---- router and experts: sigmoid scores + the shared expert's gate, squared-ReLU experts weighted at their input | Lilevik
     h = r(T, width)
     rw, rb, gw = torch.randn(E, width, device=dev), torch.randn(E, device=dev) * 0.1, torch.randn(width, device=dev)
     route = lambda v: seq_ops.moe_route(v, rw, top, score=seq_ops.ROUTE_SIGMOID, renorm=False, gate_w=gw)  # noqa: E731
-    add("sm_moe_route sigmoid + gate (T=%d, E=%d)" % (T, E), "sm_moe_route softmax + bias", _event_time(lambda: route(h)), bytes_=T * width * 2)
-    add("sm_moe_route softmax + bias (T=%d, E=%d)" % (T, E), "-", _event_time(lambda: seq_ops.moe_route(h, rw, top, bias=rb)), bytes_=T * width * 2)
+    add("sm_moe_route sigmoid + gate (T=%d, E=%d)" % (T, E), "sm_moe_route softmax + bias", _graph_time(lambda: route(h)), bytes_=T * width * 2)
+    add("sm_moe_route softmax + bias (T=%d, E=%d)" % (T, E), "-", _graph_time(lambda: seq_ops.moe_route(h, rw, top, bias=rb)), bytes_=T * width * 2)
     idx, wts, _ = route(h)
     w_up, w_gu, w_down = r(E, F, width), r(E, 2 * F, width), r(E, width, F)
     t_up = (seq_ops.tile_expert_weights(w_up, 1), seq_ops.tile_expert_weights(w_down))
@@ -866,14 +878,14 @@ def tafopel_kernel_table(width=2048, heads=16, rank=256, ff=6144, T=8192, seq=10
                                                       weight_in=True, combine=False)
     silu = lambda v, i, w_, form: seq_ops.moe_experts(v, i, w_, w_gu, w_down, inf, 1.0, form=form, tiled=t_glu, act_kind=seq_ops.ACT_SILU_GLU)  # noqa: E731
     add("sm_moe_tiles128 squared-ReLU experts (T=%d, top %d of %d, F=%d)" % (T, top, E, F), "sm_moe_tiles128 SiLU-gated experts",
-        _event_time(lambda: relu(h, idx, wts, "tiles128"), 5), flops=T * top * 4 * width * F)
-    add("sm_moe_tiles128 SiLU-gated experts (T=%d)" % T, "-", _event_time(lambda: silu(h, idx, wts, "tiles128"), 5), flops=T * top * 6 * width * F)
+        _graph_time(lambda: relu(h, idx, wts, "tiles128"), 5), flops=T * top * 4 * width * F)
+    add("sm_moe_tiles128 SiLU-gated experts (T=%d)" % T, "-", _graph_time(lambda: silu(h, idx, wts, "tiles128"), 5), flops=T * top * 6 * width * F)
     hd = h[:B].contiguous()
     idx_d, wts_d, _ = route(hd)
     touched = len(torch.unique(idx_d))
     add("sm_moe_grouped squared-ReLU experts (T=%d: decode)" % B, "sm_moe_grouped SiLU-gated experts",
-        _event_time(lambda: relu(hd, idx_d, wts_d, "grouped")), bytes_=touched * 2 * F * width * 2)
-    add("sm_moe_grouped SiLU-gated experts (T=%d: decode)" % B, "-", _event_time(lambda: silu(hd, idx_d, wts_d, "grouped")),
+        _graph_time(lambda: relu(hd, idx_d, wts_d, "grouped")), bytes_=touched * 2 * F * width * 2)
+    add("sm_moe_grouped SiLU-gated experts (T=%d: decode)" % B, "-", _graph_time(lambda: silu(hd, idx_d, wts_d, "grouped")),
         bytes_=touched * 3 * F * width * 2)
     # ---- the merged products of a parallel block (vendor GEMMs): first (scan rows + dense gate and up), last (channels + ff)
     wf, wl, av = r(2 * C + 2 * ff, width), r(width, C + ff), out
