@@ -7,9 +7,18 @@ namespace sm {
 
 constexpr int kMaxExperts = 1024, kMaxTop = 32;
 
-constexpr int kRouteTokens = 8;      // tokens per workgroup: every router row read serves all of them
+// largest value over the wave, smallest index among equals; every lane gets both
+__device__ __forceinline__ void wave_argmax(float& v, int& i) {
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+        const float ov = __shfl_xor(v, o);
+        const int oi = __shfl_xor(i, o);
+        if (ov > v || (ov == v && oi < i)) { v = ov; i = oi; }
+    }
+}
 
-template <typename T>
+// kRouteTokens = tokens per workgroup: every router row read serves all of them
+template <typename T, int kRouteTokens>
 __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h, const float* __restrict__ router_w,
                                                         int32_t* __restrict__ idx, float* __restrict__ wts, int64_t T_all, int W,
                                                         int E, int top, int groups, int keep, int score,
@@ -25,7 +34,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
     if (staged) {
         // the workgroup's token rows (one contiguous piece of h) go to LDS once; every expert's row is then read once per
         // workgroup in 16-byte pieces and meets all the tokens there
-        T* h_lds = (T*)(z_all + kRouteTokens * RS);
+        T* h_lds = (T*)(z_all + (kRouteTokens * RS + 3) / 4 * 4);
         const T* src = h + (size_t)t0 * W;
         struct alignas(sizeof(T) * 4) Pack4 { T v[4]; };
         for (int i = threadIdx.x * 4; i < nt * W; i += 1024) *(Pack4*)(h_lds + i) = *(const Pack4*)(src + i);     // W % 4 == 0
@@ -34,6 +43,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
             const float* wr = e < E ? router_w + (size_t)e * W : gate_w;
             float d[kRouteTokens];
             for (int i = 0; i < kRouteTokens; ++i) d[i] = 0.f;
+#pragma unroll 4
             for (int c = lane * 4; c < W; c += 256) {
                 const float4 wv = *(const float4*)(wr + c);
 #pragma unroll
@@ -65,8 +75,62 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
         }
     }
     __syncthreads();
+    if (groups <= 1 && E <= 256) {
+        // no groups: a wave finishes a token, lane l holding the scores of the experts l, l + 64, ...
+        for (int i = wave; i < nt; i += 4) {
+            const int64_t t = t0 + i;
+            const float* z = z_all + i * RS;
+            if (gate_w != nullptr && lane == 0) gate_out[t] = 1.f / (1.f + expf(-z[RS - 1]));
+            float s[4], c[4], mx = -INFINITY, sum = 0.f;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int e = lane + 64 * j;
+                s[j] = e < E ? z[e] + (bias ? bias[e] : 0.f) : -INFINITY;
+                mx = fmaxf(mx, s[j]);
+            }
+            if (score == SM_ROUTE_SIGMOID) {
+#pragma unroll
+                for (int j = 0; j < 4; ++j) s[j] = 1.f / (1.f + expf(-s[j]));
+            } else {
+                mx = wave_max(mx);
+#pragma unroll
+                for (int j = 0; j < 4; ++j) { s[j] = expf(s[j] - mx); sum += s[j]; }
+                const float inv = 1.f / wave_sum(sum);
+#pragma unroll
+                for (int j = 0; j < 4; ++j) s[j] *= inv;
+            }
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int e = lane + 64 * j;
+                c[j] = e < E ? s[j] + (correction ? correction[e] : 0.f) : -INFINITY;
+            }
+            float tot = 0.f, my_w = 0.f;
+            int my_e = 0;
+            for (int k = 0; k < top; ++k) {
+                float bv = -INFINITY;
+                int be = E;
+#pragma unroll
+                for (int j = 0; j < 4; ++j)
+                    if (c[j] > bv) { bv = c[j]; be = lane + 64 * j; }
+                wave_argmax(bv, be);
+                be = min(be, E - 1);
+                float w = 0.f;
+#pragma unroll
+                for (int j = 0; j < 4; ++j)
+                    if (be == lane + 64 * j) { w = s[j]; c[j] = -INFINITY; }
+                w = __shfl(w, be & 63);
+                tot += w;
+                if (lane == k) { my_w = w; my_e = be; }
+            }
+            if (lane < top) {                    // top <= 32
+                idx[(size_t)t * top + lane] = my_e;
+                wts[(size_t)t * top + lane] = my_w * (renorm ? 1.f / (tot + 1e-20f) : 1.f);
+            }
+        }
+        return;
+    }
     if (threadIdx.x >= nt) return;
-    // one thread finishes a token: E is small and the selections are sequential by nature
+    // groups (or very many experts): one thread finishes a token, the selections one after another
     const int64_t t = t0 + threadIdx.x;
     float* z = z_all + threadIdx.x * RS;
     if (gate_w != nullptr) gate_out[t] = 1.f / (1.f + expf(-z[RS - 1]));
@@ -272,13 +336,16 @@ extern "C" int sm_moe_route(int dtype, const void* h, const float* router_w, int
     }
     if (T == 0) return SM_OK;
     // the token rows of a workgroup are staged in LDS when they fit and the rows can be moved in pieces of four channels
-    const size_t scores = (size_t)kRouteTokens * (E + groups + (gate_w ? 1 : 0)) * 4;
-    const size_t rows = (size_t)kRouteTokens * W * (dtype == SM_F32 ? 4 : 2);
-    const int staged = W % 4 == 0 && scores % 16 == 0 && scores + rows <= 60 * 1024 && ((uintptr_t)h | (uintptr_t)router_w | (uintptr_t)gate_w) % 16 == 0;
-    SM_DISPATCH(dtype, "sm_moe_route",
-                hipLaunchKernelGGL(moe_route_kernel<DT>, dim3((unsigned)((T + kRouteTokens - 1) / kRouteTokens)), dim3(256),
-                                   scores + (staged ? rows : 0), as_stream(stream), (const DT*)h, router_w, idx, wts, T, W, E,
-                                   top, groups, keep, score, correction, group_top, renorm, staged, bias, gate_w, gate_out));
+    const int tok = T >= 4096 ? 8 : (T >= 1024 ? 4 : 1);       // enough workgroups for a small step
+    const size_t scores = ((size_t)tok * (E + groups + (gate_w ? 1 : 0)) * 4 + 15) / 16 * 16;
+    const size_t rows = (size_t)tok * W * (dtype == SM_F32 ? 4 : 2);
+    const int staged = W % 4 == 0 && scores + rows <= 60 * 1024 && ((uintptr_t)h | (uintptr_t)router_w | (uintptr_t)gate_w) % 16 == 0;
+#define SM_ROUTE(TOK_)                                                                                                          \
+    hipLaunchKernelGGL((moe_route_kernel<DT, TOK_>), dim3((unsigned)((T + TOK_ - 1) / TOK_)), dim3(256), scores + (staged ? rows : 0), \
+                       as_stream(stream), (const DT*)h, router_w, idx, wts, T, W, E, top, groups, keep, score, correction, group_top, \
+                       renorm, staged, bias, gate_w, gate_out)
+    SM_DISPATCH(dtype, "sm_moe_route", if (tok == 8) SM_ROUTE(8); else if (tok == 4) SM_ROUTE(4); else SM_ROUTE(1));
+#undef SM_ROUTE
     SM_CHECK_LAUNCH("sm_moe_route");
     return SM_OK;
 }

@@ -412,6 +412,36 @@ def test_experts_weighted_at_their_input_and_gated_shared_expert(device, dtype, 
                 assert left[1] is not None and left[2] is None
 
 
+@pytest.mark.parametrize("device,dtype", CASES)
+@pytest.mark.parametrize("T", [1, 37, 1501, 4103])
+@pytest.mark.parametrize("W,E,top,score,groups", [(64, 16, 4, "sigmoid", 1), (40, 70, 8, "softmax", 1), (30, 5, 5, "sigmoid", 1), (16, 200, 32, "softmax", 1),
+                                                  (24, 300, 3, "sigmoid", 1), (48, 12, 3, "softmax", 4)])
+def test_router_step_sizes_and_scores(device, dtype, T, W, E, top, score, groups):
+    """Steps of one token to thousands (the kernel takes different numbers of tokens per workgroup), more experts than lanes,
+    both scores, with and without groups, biases, corrections that steer the choice, renormalised and plain weights."""
+    g = gen(T + E)
+    h = rnd(g, T, W, dtype=dtype)
+    rw, bias, corr, gw = rnd(g, E, W, s=2 * W ** -0.5), rnd(g, E, s=0.3), rnd(g, E, s=0.2), rnd(g, W, s=W ** -0.5)
+    z = h.to(F64) @ rw.to(F64).T + bias.to(F64)
+    s = torch.sigmoid(z) if score == "sigmoid" else torch.softmax(z, -1)
+    c = s + corr.to(F64)
+    if groups > 1:
+        best = c.view(T, groups, -1).max(-1).values.topk(2, -1).indices
+        keep = torch.zeros(T, groups, dtype=torch.bool).scatter_(1, best, True)
+        c = c.masked_fill(~keep.repeat_interleave(E // groups, 1), float("-inf"))
+    for renorm in (False, True):
+        idx, wts, gate = seq_ops.moe_route(h.to(device), rw.to(device), top, groups, 2 if groups > 1 else 1,
+                                           seq_ops.ROUTE_SIGMOID if score == "sigmoid" else seq_ops.ROUTE_SOFTMAX, corr.to(device), 1, renorm,
+                                           bias.to(device), gw.to(device))
+        idx, wts = idx.cpu().long(), wts.cpu().to(F64)
+        assert all(len(set(r)) == top for r in idx[:50].tolist())
+        chosen = c.gather(1, idx)                          # (near-ties may fall either way: the choice scores decide)
+        near(chosen.sort(-1).values, c.topk(top, -1).values.sort(-1).values, torch.float32, f32=2e-5)
+        w = s.gather(1, idx)
+        near(wts, w / w.sum(-1, keepdim=True) if renorm else w, torch.float32, f32=5e-5)
+        near(gate, torch.sigmoid(h.to(F64) @ gw.to(F64)), torch.float32, f32=2e-5)
+
+
 @pytest.mark.gpu
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("act", ["gelu", "clamped_glu", "silu_glu", "gelu_tanh_glu", "relu_sq"])
