@@ -19,10 +19,10 @@ of its own, a paged key and value cache and the pooled caches beside them, and p
 import re
 
 import torch
-import torch.nn.functional as F
 from torch import nn
 
 from nanovllm import hy_ops, seq_ops
+from nanovllm.layers.f32_product import F32Product
 from nanovllm.layers.feedforward import RoutedExperts
 from nanovllm.layers.latent_attention import LatentAttention
 from nanovllm.layers.rotary_attention import PagedRotaryAttention
@@ -97,7 +97,7 @@ class GalupelForCausalLM(nn.Module):
             layers.append(GalupelLayer(cfg, spec, layers))
         self.layers = nn.ModuleList(layers)
         self.final_norm = nn.Parameter(torch.ones(W), requires_grad=False)
-        self._f32_out = None       # whether the vendor GEMM writes float32 from 16-bit operands for the head's shape
+        self.logits_product = F32Product()
 
     # ------------------------------------------------------------------ checkpoint names
     _SIMPLE = {"norm1": "norm1", "norm2": "norm2", "mix.o": "mixer.o_proj", "mix.q.norm": "mixer.q_head_norm",
@@ -238,18 +238,5 @@ class GalupelForCausalLM(nn.Module):
     def compute_logits(self, hidden_states):
         """float32 logits of the given rows: products with the embedding table (float32 accumulation AND output), times
         logit_scale, soft-capped."""
-        if hidden_states.dtype == torch.float32:
-            out = F.linear(hidden_states, self.embed)
-        else:
-            out = None
-            if hidden_states.is_cuda and self._f32_out is not False:
-                try:
-                    out = torch.mm(hidden_states, self.embed.t(), out_dtype=torch.float32)
-                    self._f32_out = True
-                except RuntimeError:
-                    if self._f32_out:          # it has worked before: this is another fault
-                        raise
-                    self._f32_out = False      # no such GEMM for this shape: the same sums from widened operands
-            if out is None:
-                out = F.linear(hidden_states.float(), self.embed.float())
+        out = self.logits_product(hidden_states, self.embed)
         return hy_ops.scale_softcap_(out.contiguous(), self.cfg.logit_scale, self.cfg.logit_softcap)

@@ -21,11 +21,11 @@ table) and, per state slot, the float32 state of every lightning layer."""
 import re
 
 import torch
-import torch.nn.functional as F
 from torch import nn
 
 from nanovllm import hy_ops
 from nanovllm.layers.dyn_tanh import DynTanh
+from nanovllm.layers.f32_product import F32Product
 from nanovllm.layers.feedforward import RoutedExperts
 from nanovllm.layers.latent_attention import LatentAttention
 from nanovllm.layers.lightning import LightningAttention
@@ -87,7 +87,7 @@ class LilevikForCausalLM(nn.Module):
         self.embed = nn.Parameter(torch.empty(cfg.vocab_size, W), requires_grad=False)
         self.layers = nn.ModuleList([LilevikLayer(cfg, spec) for spec in cfg.layers])
         self.final_norm = DynTanh(W)
-        self._f32_out = None       # whether the vendor GEMM writes float32 from 16-bit operands for the head's shape
+        self.logits_product = F32Product()
 
     # ------------------------------------------------------------------ checkpoint names
     _SIMPLE = {"mix.o": "mixer.o_proj", "mix.q.norm": "mixer.q_norm", "mix.k.norm": "mixer.k_norm", "mix.pb": "mixer.head_bias",
@@ -256,15 +256,4 @@ class LilevikForCausalLM(nn.Module):
 
     def compute_logits(self, hidden_states):
         """float32 logits of the given rows: products with the embedding table, float32 accumulation AND output."""
-        if hidden_states.dtype == torch.float32:
-            return F.linear(hidden_states, self.embed)
-        if hidden_states.is_cuda and self._f32_out is not False:
-            try:
-                out = torch.mm(hidden_states, self.embed.t(), out_dtype=torch.float32)
-                self._f32_out = True
-                return out
-            except RuntimeError:
-                if self._f32_out:          # it has worked before: this is another fault
-                    raise
-                self._f32_out = False      # no such GEMM for this shape: the same sums from widened operands
-        return F.linear(hidden_states.float(), self.embed.float())
+        return self.logits_product(hidden_states, self.embed)

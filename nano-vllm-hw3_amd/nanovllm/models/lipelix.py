@@ -22,6 +22,7 @@ from torch import nn
 
 from nanovllm import hy_ops, seq_ops
 from nanovllm.layers.delta_rule import GeneralDelta
+from nanovllm.layers.f32_product import F32Product
 from nanovllm.layers.feedforward import ReluSquaredMLP
 from nanovllm.layers.gated_sublayer import GatedPort
 from nanovllm.layers.rotary_attention import PagedRotaryAttention
@@ -99,7 +100,7 @@ class LipelixForCausalLM(nn.Module):
         self.layers = nn.ModuleList([LipelixLayer(cfg, spec) for spec in cfg.layers])
         self.final_norm = nn.Parameter(torch.ones(W), requires_grad=False)
         self.head = nn.Parameter(torch.empty(cfg.vocab_size, W), requires_grad=False)
-        self._f32_out = None       # whether the vendor GEMM writes float32 from 16-bit operands for the head's shape
+        self.logits_product = F32Product()
         # the first layer that mixes values gives them; it blends nothing itself
         self.v_source = next((i for i, l in enumerate(self.layers) if getattr(l.mixer, "v_mix", False)), None)
 
@@ -267,15 +268,4 @@ class LipelixForCausalLM(nn.Module):
 
     def compute_logits(self, hidden_states):
         """float32 logits of the given rows: products of the stored values, float32 accumulation AND output."""
-        if hidden_states.dtype == torch.float32:
-            return F.linear(hidden_states, self.head)
-        if hidden_states.is_cuda and self._f32_out is not False:
-            try:
-                out = torch.mm(hidden_states, self.head.t(), out_dtype=torch.float32)
-                self._f32_out = True
-                return out
-            except RuntimeError:
-                if self._f32_out:          # it has worked before: this is another fault
-                    raise
-                self._f32_out = False      # no such GEMM for this shape: the same sums from widened operands
-        return F.linear(hidden_states.float(), self.head.float())
+        return self.logits_product(hidden_states, self.head)

@@ -15,11 +15,11 @@ decoded tokens in one batch.  Residual streams, norms, softmax and router scores
 import re
 
 import torch
-import torch.nn.functional as F
 from torch import nn
 
 from nanovllm import seq_ops
 from nanovllm.layers.canon import CausalTaps
+from nanovllm.layers.f32_product import F32Product
 from nanovllm.layers.feedforward import ClampedGLU, PolyNormMLP, RoutedExperts
 from nanovllm.layers.latent_attention import LatentAttention
 from nanovllm.layers.streams import StreamPort
@@ -94,7 +94,7 @@ class PasizenForCausalLM(nn.Module):
         self.head = nn.Parameter(torch.empty(cfg.vocab_size, W), requires_grad=False)
         self.run_order = list(cfg.run_order)
         self.sum_streams = torch.ones(cfg.streams, dtype=torch.float32)
-        self._f32_out = None       # whether the vendor GEMM writes float32 from 16-bit operands for the head's shape
+        self.logits_product = F32Product()
 
     # ------------------------------------------------------------------ checkpoint names
     _SIMPLE = {"norm1": "norm1", "norm2": "norm2", "canon1": "canon.weight", "mix.dkv.norm": "mixer.latent_norm",
@@ -249,15 +249,4 @@ class PasizenForCausalLM(nn.Module):
 
     def compute_logits(self, hidden_states):
         """float32 logits of the given rows: products of the stored values, float32 accumulation AND output."""
-        if hidden_states.dtype == torch.float32:
-            return F.linear(hidden_states, self.head)
-        if hidden_states.is_cuda and self._f32_out is not False:
-            try:
-                out = torch.mm(hidden_states, self.head.t(), out_dtype=torch.float32)
-                self._f32_out = True
-                return out
-            except RuntimeError:
-                if self._f32_out:          # it has worked before: this is another fault
-                    raise
-                self._f32_out = False      # no such GEMM for this shape: the same sums from widened operands
-        return F.linear(hidden_states.float(), self.head.float())
+        return self.logits_product(hidden_states, self.head)
