@@ -4,11 +4,12 @@ Three libraries, each from its own folder of translation units, so that a model 
   qlinear  csrc/*.hip         -> nanovllm/_lib/libqlinear.so   (quantized linears, Qwen3 operators, attention)
   seqmix   csrc/seqmix/*.hip  -> nanovllm/_lib/libseqmix.so    (multi-stream residuals, short convolutions, latent
                                                                 attention with or without a rotated part and a window,
-                                                                PolyNorm / clamped GLU / GELU experts, expert routing)
-  hymix    csrc/hymix/*.hip   -> nanovllm/_lib/libhymix.so     (gated, grouped-norm and tanh-norm residuals, token shift,
+                                                                PolyNorm / gated / GELU / squared-ReLU feed-forwards,
+                                                                expert routing)
+  hymix    csrc/hymix/*.hip   -> nanovllm/_lib/libhymix.so     (gated, grouped-norm, tanh-norm and layer-norm residuals, token shift,
                                                                 attention with sinks, windows, pooled blocks, chunked
-                                                                masks and sigmoid weights over a paged cache, delta-rule
-                                                                and constant-decay recurrences)
+                                                                masks and sigmoid weights over a paged cache, delta-rule,
+                                                                constant-decay and selective-scan recurrences)
 ``python build.py [--force] [qlinear|seqmix|hymix]`` builds one of them, or all without a name."""
 import os
 import shutil
